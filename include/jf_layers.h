@@ -17,7 +17,7 @@ extern "C" {
 #endif
 
 #define JL_API __attribute__((visibility("default")))
-#define JL_VERSION 124
+#define JL_VERSION 125
 #define JL_OK 0
 #define JL_E_INVALID (-1)
 #define JL_E_LAUNCH (-3)
@@ -57,6 +57,7 @@ JL_API int jl_scaled_add_norms(float *x, const jl_addend *addends, int32_t n_add
 #define JL_ACT_CLAMPED_SWISH 1
 #define JL_ACT_SILU 2             /* act(g) = g sigmoid(g), lin(u) = u */
 #define JL_ACT_GELU_ERF 3         /* act(g) = 0.5 g (1 + erf(g / sqrt 2)), lin(u) = u */
+#define JL_ACT_SIGMOID 4          /* gates only (jl_gated_norm) */
 #define JL_ACT_NONE (-1)          /* where an activation is optional (jl_short_conv) */
 JL_API int jl_gated_act(const void *z, int dtype, int64_t N, int64_t ld, int32_t g_col, int32_t u_col, int32_t F, int32_t kind, float limit,
                         float alpha, float shift, const void *row_gate, int64_t rg_ld, void *out, void *stream);
@@ -64,10 +65,12 @@ JL_API int jl_gated_act(const void *z, int dtype, int64_t N, int64_t ld, int32_t
 /* Whole-projection query / key norm + cache append.  proj [N, ld] holds q (H*D columns at q_col), k (G*D at k_col) and v (G*Dv at
  * v_col).  q_out [N, H*D] = rms_norm(q) * wq over ALL H*D columns at once; the key is normalised the same way over G*D with wk and
  * stored at k_cache[slot[n]] ([pool tokens, G*D]); v is stored as it is at v_cache[slot[n]] ([pool tokens, G*Dv]).  slot < 0 skips
- * the stores. */
+ * the stores.  With rot_dims > 0 the first rot_dims dimensions of every head of q and k are rotated by the position pos[n] behind the norm
+ * (`pairing` JL_ROT_HALVES / JL_ROT_NEIGHBOURS, angles from the cos / sin tables [positions, rot_dims/2] float). */
 JL_API int jl_qk_norm_append(const void *proj, int dtype, int64_t N, int64_t ld, int32_t q_col, int32_t k_col, int32_t v_col,
                              int32_t H, int32_t G, int32_t D, int32_t Dv, const void *wq, const void *wk, float eps, void *q_out,
-                             void *k_cache, void *v_cache, const int64_t *slot, void *stream);
+                             void *k_cache, void *v_cache, const int64_t *slot, int32_t rot_dims, int32_t pairing, const int32_t *pos,
+                             const float *cos_t, const float *sin_t, void *stream);
 
 /* Attention over the paged pool with a sliding window that keeps the first tokens, a bucketed distance bias and mixed heads:
  *   visible(i, j) = j <= i and (i - j < window or j < keep_first)
@@ -94,6 +97,10 @@ typedef struct {
     int32_t out_dtype;            /* dtype of `out` when it differs from `dtype`: JL_OUT_F32 = float outputs from bfloat16 inputs     */
     const float *sink;            /* float [H] or null: one more term exp(sink[g]) in head g's softmax denominator                    */
     int32_t gate_heads;           /* != 0: `gate` holds one number per head ([N, H]) instead of one per output element                */
+    int32_t chunk;                /* > 0: visible(i, j) = j <= i and i / chunk == j / chunk (no window, no kept first tokens)          */
+    float softcap;                /* > 0: scores pass softcap * tanh(s / softcap) behind scale and bias (the sink does not)            */
+    float out_scale;              /* the outputs times this (1 when there is nothing to scale)                                        */
+    int64_t out_ld;               /* row stride of `out` in elements (0: H*Dv)                                                       */
 } jl_attn_args;
 #define JL_OUT_SAME 0
 #define JL_OUT_F32 2
@@ -148,6 +155,22 @@ JL_API int jl_softcap(float *z, int64_t total, float cap, void *stream);
 JL_API int jl_norm_add(float *x, const void *y, int y_dtype, const float *g, float eps, void *out, int out_dtype, int64_t N, int32_t W,
                        void *stream);
 
+/* A layer with a norm in front of and behind each sublayer — the norm on a sublayer's OUTPUT, the residual update and the NEXT sublayer's
+ * norm in one launch:
+ *   x_out[n] = x_in[n] + y[n] / sqrt(mean(y[n]^2) + eps) * w_post + add_row          (y null: no sublayer output; add_row float [W] or null)
+ *   out[n]   = x_out[n] / sqrt(mean(x_out[n]^2) + eps) * w_next, or x_out[n] itself (plain != 0), in `dtype`, rows out_ld elements apart
+ * x_in, x_out float [N, W] (may be the same; neither y nor add_row: nothing is stored and `out` comes from x_in); y of y_dtype; w_post, w_next
+ * float [W]; out may be null. */
+JL_API int jl_sandwich_norm(const float *x_in, float *x_out, const void *y, int y_dtype, const float *w_post, const float *add_row, float eps,
+                            const float *w_next, void *out, int dtype, int64_t out_ld, int32_t plain, int64_t N, int32_t W, void *stream);
+
+/* Norm and gate on a recurrent mixer's float output raw [N, C], over `parts` equal parts of the row (each by its own root mean square):
+ *   gate_first != 0:  v = raw * act(gate), out = v / sqrt(mean(v^2) + eps) * w * scale
+ *   gate_first == 0:  out = raw / sqrt(mean(raw^2) + eps) * w * act(gate) * scale
+ * gate [N, C] of `dtype`, rows gate_ld apart; w float [C]; act JL_ACT_SILU or JL_ACT_SIGMOID; out [N, C] of `dtype`, rows out_ld apart. */
+JL_API int jl_gated_norm(const float *raw, const void *gate, int dtype, int64_t gate_ld, const float *w, float eps, int32_t act, int32_t gate_first,
+                         float scale, void *out, int64_t out_ld, int64_t N, int32_t C, int32_t parts, void *stream);
+
 /* Polynomial activation with unit-RMS powers: out = c0 n(z) + c1 n(z^2) + c2 n(z^3) + c3, powers element by element,
  * n(u) = u / sqrt(mean(u^2) + eps) over the row's F values.  z, out [N, F] of `dtype`; coef four floats. */
 JL_API int jl_polynorm(const void *z, int dtype, int64_t N, int32_t F, const float *coef, float eps, void *out, void *stream);
@@ -164,13 +187,13 @@ JL_API int jl_causal_conv(const float *x, const void *w, int dtype, const int32_
                           int64_t N, int32_t W, int32_t taps, void *out, void *stream);
 JL_API int jl_causal_conv_carry(const float *x, const int32_t *seq, int32_t B, float *tail, int32_t W, int32_t taps, void *stream);
 
-/* Short causal convolution over time of a column range of a product, with an activation and no residual:
- *   out[t, c] = act(sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start)
- * x [N, ld] and w [C, taps] of `dtype`, out float [N, C]; act JL_ACT_SILU or JL_ACT_NONE; taps <= 8.  tail float [slots, taps - 1, C] as for
+/* Short causal convolution over time of a column range of a product, with an optional bias and an activation and no residual:
+ *   out[t, c] = act(bias[c] + sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start)
+ * x [N, ld], w [C, taps] and bias [C] (null: none) of `dtype`, out [N, C] float or of `dtype` (`out_dtype`); act JL_ACT_SILU or JL_ACT_NONE; taps <= 8.  tail float [slots, taps - 1, C] as for
  * jl_causal_conv (the INPUTS at the positions before the step); it is moved on here as well — for requests with one row in the launch
  * itself, for the others (max_count > 1) by a second launch enqueued behind it. */
-JL_API int jl_short_conv(const void *x, int dtype, int64_t ld, int32_t col, const void *w, const int32_t *row_req, const int32_t *seq, int32_t B,
-                         int32_t max_count, float *tail, int64_t N, int32_t C, int32_t taps, int32_t act, float *out, void *stream);
+JL_API int jl_short_conv(const void *x, int dtype, int64_t ld, int32_t col, const void *w, const void *bias, const int32_t *row_req, const int32_t *seq, int32_t B,
+                         int32_t max_count, float *tail, int64_t N, int32_t C, int32_t taps, int32_t act, void *out, int out_dtype, void *stream);
 
 /* Per-head query / key stage for attention with M score maps per head: rotation, norm, query temperature, cache append.  proj
  * [N, ld] holds q (H heads x M maps x D at q_col, head by head), k (G x M x D at k_col) and v (G x Dv at v_col).  With rot_dims > 0
@@ -252,6 +275,25 @@ JL_API int jl_delta_rule(const void *qkv, int qkv_dtype, int64_t qkv_ld, int32_t
                          int64_t ld, int32_t a_col, int32_t b_col, int32_t g_col, const float *A_log, const float *dt_bias, const float *norm_w,
                          const int32_t *seq, int32_t B, int64_t N, int32_t H, int32_t G, int32_t D, int32_t Dv, float unit_eps, float q_scale, float eps,
                          float *state, float *raw, void *out, void *stream);
+
+/* Linear recurrence with one decay per head (and token) over the ragged batch, state carried in float — lightning attention and the
+ * state-space duality of Mamba-2 in one form.  Per head h (q / k head c = h / (H / G)) and token t:
+ *   S_t = a_t S_(t-1) + k_t (u_t v_t)^T,   o_t = S_t^T q_t + skip_h v_t            (S [D, Dv]; the read-out sees the token's own write)
+ * fixed decays (`decay` float [H]): a_t = decay[h], u_t = 1;  otherwise u_t = softplus(dt_h(t) + dt_bias[h]), a_t = exp(-exp(A_log[h]) u_t).
+ * q, k (G*D columns each) and v (H*Dv) lie in src [N, ld] of `dtype` and pass `act` (JL_ACT_SILU or JL_ACT_NONE) on the way in; dt (H columns)
+ * in dt [N, dt_ld] of `dtype`; skip float [H] or null.  state [slots, H, D, Dv] float: a request with pos0 == 0 starts from zero (its
+ * slot's old content is ignored); the final state is written back.  out float [N, H*Dv].  D <= 256.
+ * `chunks` 0: every request's rows in one scan.  `chunks` > 0 (bfloat16, long portions): the portions are cut into `chunks` pieces that
+ * run side by side on the matrix cores — chunk_rec [chunks, 4] int32 {row0, count, pos0, piece}, req [B, 4] int32 {first piece, pieces,
+ * pos0, slot}, scratch of chunks * H * (D * Dv + 1) floats; sizes as jl_linear_scan_chunked_ok accepts them. */
+typedef struct {
+    const void *src; const void *dt; const float *decay; const float *A_log; const float *dt_bias; const float *skip;
+    const int32_t *seq; float *state; float *out; const int32_t *chunk_rec; const int32_t *req; float *scratch;
+    int64_t ld, dt_ld, N;
+    int32_t q_col, k_col, v_col, dt_col, dtype, act, B, H, G, D, Dv, chunks;
+} jl_scan_args;
+JL_API int jl_linear_scan(const jl_scan_args *a, void *stream);
+JL_API int jl_linear_scan_chunked_ok(int dtype, int32_t D, int32_t Dv);
 
 /* Router of a mixture of experts over float logits [N, E]; ids [N, top] int32, weights [N, top] float.
  *   JL_ROUTE_SIGMOID:        s = sigmoid(logits); the `top` experts with the largest s + correction are chosen (ties: lowest

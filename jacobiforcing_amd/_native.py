@@ -231,9 +231,9 @@ def raise_state_error(code: int, what: str, aux: int = 0):
 
 # ---- libjf_layers.so (include/jf_layers.h): layer kernels of the models whose forward is not stock PyTorch ----------------------------
 JL_F32, JL_BF16 = 0, 1
-JL_VERSION = 124                 # include/jf_layers.h: a library of another version is not called (its signatures may differ)
+JL_VERSION = 125                 # include/jf_layers.h: a library of another version is not called (its signatures may differ)
 JL_OUT_SAME, JL_OUT_F32 = 0, 2
-JL_ACT_GELU_TANH, JL_ACT_CLAMPED_SWISH, JL_ACT_SILU, JL_ACT_GELU_ERF, JL_ACT_NONE = 0, 1, 2, 3, -1
+JL_ACT_GELU_TANH, JL_ACT_CLAMPED_SWISH, JL_ACT_SILU, JL_ACT_GELU_ERF, JL_ACT_SIGMOID, JL_ACT_NONE = 0, 1, 2, 3, 4, -1
 JL_ROUTE_SIGMOID, JL_ROUTE_SOFTMAX_RENORM, JL_ROUTE_TOP_SOFTMAX = 0, 1, 2
 JL_ROT_HALVES, JL_ROT_NEIGHBOURS = 0, 1
 JL_MOE_UP_RELU2, JL_MOE_DOWN, JL_MOE_UP_PLAIN = 0, 1, 2
@@ -246,7 +246,14 @@ class AttnArgs(C.Structure):
                 ("bt_stride", _i32), ("n_tiles", _i32), ("lut_len", _i32), ("page_size", _i32), ("H", _i32), ("G", _i32), ("D", _i32),
                 ("Dv", _i32), ("window", _i32), ("keep_first", _i32), ("TQ", _i32), ("dtype", _i32), ("scale", _f32),
                 ("splits", _i32), ("n_rows", _i32), ("scratch", _vp), ("q_pack", _vp), ("k_ld", _i64), ("v_ld", _i64), ("Gv", _i32),
-                ("out_dtype", _i32), ("sink", _vp), ("gate_heads", _i32)]
+                ("out_dtype", _i32), ("sink", _vp), ("gate_heads", _i32), ("chunk", _i32), ("softcap", _f32), ("out_scale", _f32), ("out_ld", _i64)]
+
+
+class ScanArgs(C.Structure):
+    """jl_scan_args (include/jf_layers.h)."""
+    _fields_ = [(k, _vp) for k in ("src", "dt", "decay", "A_log", "dt_bias", "skip", "seq", "state", "out", "chunk_rec", "req", "scratch")] + \
+               [(k, _i64) for k in ("ld", "dt_ld", "N")] + \
+               [(k, _i32) for k in ("q_col", "k_col", "v_col", "dt_col", "dtype", "act", "B", "H", "G", "D", "Dv", "chunks")]
 
 
 class Addend(C.Structure):
@@ -259,7 +266,8 @@ _LAYER_SIGNATURES = {
     "jl_last_error": (C.c_char_p, []),
     "jl_embed_scale": (C.c_int, [_vp, C.c_int, _vp, _i64, _i32, _f32, _vp, _vp, _vp]),
     "jl_add_rmsnorm": (C.c_int, [_vp, _vp, C.c_int, _i32, _vp, _vp, _f32, _vp, C.c_int, _i64, _i32, _vp]),
-    "jl_qk_norm_append": (C.c_int, [_vp, C.c_int, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _vp]),
+    "jl_qk_norm_append": (C.c_int, [_vp, C.c_int, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32,
+                                    _vp, _vp, _vp, _vp]),
     "jl_attn_window": (C.c_int, [C.POINTER(AttnArgs), _vp]),
     "jl_attn_scratch_floats": (_i64, [_i32, _i32, _i32, _i32, _i32]),
     "jl_attn_tile_rows": (C.c_int, [C.c_int, _i32, _i32, _i32, _i32, _i64, _i64]),
@@ -283,7 +291,11 @@ _LAYER_SIGNATURES = {
                                     _vp]),
     "jl_token_shift": (C.c_int, [_vp, _vp, _vp, _vp, _vp, _i64, _i32, _vp, C.c_int, _vp]),
     "jl_softcap": (C.c_int, [_vp, _i64, _f32, _vp]),
-    "jl_short_conv": (C.c_int, [_vp, C.c_int, _i64, _i32, _vp, _vp, _vp, _i32, _i32, _vp, _i64, _i32, _i32, _i32, _vp, _vp]),
+    "jl_short_conv": (C.c_int, [_vp, C.c_int, _i64, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _vp, _i64, _i32, _i32, _i32, _vp, C.c_int, _vp]),
+    "jl_sandwich_norm": (C.c_int, [_vp, _vp, _vp, C.c_int, _vp, _vp, _f32, _vp, _vp, C.c_int, _i64, _i32, _i64, _i32, _vp]),
+    "jl_gated_norm": (C.c_int, [_vp, _vp, C.c_int, _i64, _vp, _f32, _i32, _i32, _f32, _vp, _i64, _i64, _i32, _i32, _vp]),
+    "jl_linear_scan": (C.c_int, [C.POINTER(ScanArgs), _vp]),
+    "jl_linear_scan_chunked_ok": (C.c_int, [C.c_int, _i32, _i32]),
     "jl_delta_rule": (C.c_int, [_vp, C.c_int, _i64, _i32, _i32, _i32, _vp, C.c_int, _i64, _i32, _i32, _i32, _vp, _vp, _vp, _vp, _i32, _i64, _i32, _i32,
                                 _i32, _i32, _f32, _f32, _f32, _vp, _vp, _vp, _vp]),
     "jl_heads_gate": (C.c_int, [_vp, _vp, _i64, C.c_int, _i64, _i32, _i32, _vp, _vp]),
@@ -298,7 +310,7 @@ _LAYER_SIGNATURES = {
 }
 LAYER_SYMBOLS = tuple(_LAYER_SIGNATURES)
 # which library a symbol lives in (jacobiforcing_amd/_build.py: LAYER_GROUPS); both carry their own jl_version / jl_last_error
-_SEQ_SYMBOLS = ("jl_retention", "jl_retention_join", "jl_delta_rule", "jl_moe_route", "jl_moe_group", "jl_moe_tile_rows", "jl_moe_gemm", "jl_moe_gemm_gated")
+_SEQ_SYMBOLS = ("jl_retention", "jl_retention_join", "jl_delta_rule", "jl_linear_scan", "jl_linear_scan_chunked_ok", "jl_moe_route", "jl_moe_group", "jl_moe_tile_rows", "jl_moe_gemm", "jl_moe_gemm_gated")
 
 
 class _LayerLibs:

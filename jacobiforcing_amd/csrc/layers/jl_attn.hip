@@ -5,11 +5,22 @@
 #include <type_traits>
 
 // ---- whole-projection q / k norm + append: one workgroup per token ------------------------------------------------------------
+// The norm runs over all heads of q (and of k) together; the rotation by position then turns each head's first rot_dims dimensions.
+// element d of a head after norm and rotation, from a reader of the normalised elements of that head
+template <typename F>
+__device__ __forceinline__ float qk_turned(F x, int d, int rot_dims, int pairing, const float *ct, const float *sn) {
+    if (d >= rot_dims) return x(d);
+    const int half = rot_dims >> 1;
+    if (pairing == JL_ROT_NEIGHBOURS) return d & 1 ? x(d) * ct[d >> 1] + x(d - 1) * sn[d >> 1] : x(d) * ct[d >> 1] - x(d + 1) * sn[d >> 1];
+    return d < half ? x(d) * ct[d] - x(d + half) * sn[d] : x(d) * ct[d - half] + x(d - half) * sn[d - half];
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void qk_norm_append_kernel(const T *__restrict__ proj, int64_t ld, int q_col, int k_col, int v_col,
-                                                              int HD, int GD, int GDv, const T *__restrict__ wq, const T *__restrict__ wk,
+                                                              int HD, int GD, int GDv, int D, const T *__restrict__ wq, const T *__restrict__ wk,
                                                               float eps, T *__restrict__ q_out, T *__restrict__ k_cache,
-                                                              T *__restrict__ v_cache, const int64_t *__restrict__ slot) {
+                                                              T *__restrict__ v_cache, const int64_t *__restrict__ slot, int rot_dims, int pairing,
+                                                              const int32_t *__restrict__ pos, const float *__restrict__ cos_t, const float *__restrict__ sin_t) {
     __shared__ float red[16];
     const int64_t n = blockIdx.x;
     const T *row = proj + n * ld;
@@ -19,23 +30,124 @@ __global__ __launch_bounds__(256) void qk_norm_append_kernel(const T *__restrict
     sq = block_sum_f32(sq, red);
     sk = block_sum_f32(sk, red);
     const float rq = 1.0f / sqrtf(sq / (float)HD + eps), rk = 1.0f / sqrtf(sk / (float)GD + eps);
-    for (int c = threadIdx.x; c < HD; c += 256) st_f(q_out + n * HD + c, ld_f(row + q_col + c) * rq * ld_f(wq + c));
+    const float *ct = rot_dims ? cos_t + (int64_t)pos[n] * (rot_dims >> 1) : nullptr, *sn = rot_dims ? sin_t + (int64_t)pos[n] * (rot_dims >> 1) : nullptr;
+    for (int c = threadIdx.x; c < HD; c += 256) {
+        const int c0 = c - c % D;
+        auto x = [&](int d) { return ld_f(row + q_col + c0 + d) * rq * ld_f(wq + c0 + d); };
+        st_f(q_out + n * HD + c, qk_turned(x, c - c0, rot_dims, pairing, ct, sn));
+    }
     const int64_t sl = slot[n];
     if (sl < 0) return;
-    for (int c = threadIdx.x; c < GD; c += 256) st_f(k_cache + sl * GD + c, ld_f(row + k_col + c) * rk * ld_f(wk + c));
+    for (int c = threadIdx.x; c < GD; c += 256) {
+        const int c0 = c - c % D;
+        auto x = [&](int d) { return ld_f(row + k_col + c0 + d) * rk * ld_f(wk + c0 + d); };
+        st_f(k_cache + sl * GD + c, qk_turned(x, c - c0, rot_dims, pairing, ct, sn));
+    }
     for (int c = threadIdx.x; c < GDv; c += 256) v_cache[sl * GDv + c] = row[v_col + c];
+}
+
+// The same four elements at a time (D, columns and strides in multiples of four, neighbouring pairs or no rotation): a thread keeps its
+// part of q and of k in registers between the sum of squares and the output.
+template <typename T, int QI, int KI>                                    // HD <= 1024 * QI, GD <= 1024 * KI
+__global__ __launch_bounds__(256) void qk_norm_append_vec_kernel(const T *__restrict__ proj, int64_t ld, int q_col, int k_col, int v_col,
+                                                                  int HD, int GD, int GDv, int D, const T *__restrict__ wq, const T *__restrict__ wk,
+                                                                  float eps, T *__restrict__ q_out, T *__restrict__ k_cache,
+                                                                  T *__restrict__ v_cache, const int64_t *__restrict__ slot, int rot_dims,
+                                                                  const int32_t *__restrict__ pos, const float *__restrict__ cos_t, const float *__restrict__ sin_t) {
+    __shared__ float red[2][4];
+    const int64_t n = blockIdx.x;
+    const T *row = proj + n * ld;
+    const int64_t sl = slot[n];
+    const int p = rot_dims ? pos[n] : 0;
+    float q[QI][4], k[KI][4], sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int i = 0; i < QI; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 4;
+        if (c < HD) {
+            ld4_f(row + q_col + c, q[i]);
+            sq += q[i][0] * q[i][0] + q[i][1] * q[i][1] + q[i][2] * q[i][2] + q[i][3] * q[i][3];
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < KI; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 4;
+        if (c < GD) {
+            ld4_f(row + k_col + c, k[i]);
+            sk += k[i][0] * k[i][0] + k[i][1] * k[i][1] + k[i][2] * k[i][2] + k[i][3] * k[i][3];
+        }
+    }
+    if (sl >= 0)
+        for (int c = threadIdx.x * 4; c < GDv; c += 1024) {
+            float v[4];
+            ld4_f(row + v_col + c, v);
+            st4_f(v_cache + sl * GDv + c, v);
+        }
+    sq = wave_sum_f32(sq);
+    sk = wave_sum_f32(sk);
+    if ((threadIdx.x & 63) == 0) { red[0][threadIdx.x >> 6] = sq; red[1][threadIdx.x >> 6] = sk; }
+    __syncthreads();
+    sq = (red[0][0] + red[0][1]) + (red[0][2] + red[0][3]);
+    sk = (red[1][0] + red[1][1]) + (red[1][2] + red[1][3]);
+    const float rq = 1.0f / sqrtf(sq / (float)HD + eps), rk = 1.0f / sqrtf(sk / (float)GD + eps);
+    auto finish = [&](float (&x)[4], int c, float r, const T *w) {
+        float g[4];
+        ld4_f(w + c, g);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) x[i] *= r * g[i];
+        const int d = c % D;
+        if (d < rot_dims) {                                             // rot_dims is a multiple of four: two whole pairs
+            const int64_t a = (int64_t)p * (rot_dims >> 1) + (d >> 1);
+#pragma unroll
+            for (int i = 0; i < 2; ++i) {
+                const float cs = cos_t[a + i], sn = sin_t[a + i], u = x[2 * i], v = x[2 * i + 1];
+                x[2 * i] = u * cs - v * sn;
+                x[2 * i + 1] = v * cs + u * sn;
+            }
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < QI; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 4;
+        if (c < HD) { finish(q[i], c, rq, wq); st4_f(q_out + n * HD + c, q[i]); }
+    }
+    if (sl < 0) return;
+#pragma unroll
+    for (int i = 0; i < KI; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 4;
+        if (c < GD) { finish(k[i], c, rk, wk); st4_f(k_cache + sl * GD + c, k[i]); }
+    }
 }
 
 extern "C" int jl_qk_norm_append(const void *proj, int dtype, int64_t N, int64_t ld, int32_t q_col, int32_t k_col, int32_t v_col,
                                  int32_t H, int32_t G, int32_t D, int32_t Dv, const void *wq, const void *wk, float eps, void *q_out,
-                                 void *k_cache, void *v_cache, const int64_t *slot, void *stream) {
+                                 void *k_cache, void *v_cache, const int64_t *slot, int32_t rot_dims, int32_t pairing, const int32_t *pos,
+                                 const float *cos_t, const float *sin_t, void *stream) {
     if (N <= 0) return JL_OK;
     if (!proj || !wq || !wk || !q_out || !k_cache || !v_cache || !slot) return jl_fail(JL_E_INVALID, "jl_qk_norm_append: null pointer");
-    if (H <= 0 || G <= 0 || D <= 0 || Dv <= 0 || q_col + H * D > ld || k_col + G * D > ld || v_col + G * Dv > ld)
+    if (H <= 0 || G <= 0 || D <= 0 || Dv <= 0 || q_col + (int64_t)H * D > ld || k_col + (int64_t)G * D > ld || v_col + (int64_t)G * Dv > ld)
         return jl_fail(JL_E_INVALID, "jl_qk_norm_append: columns do not fit the row stride");
-    JL_DISPATCH(dtype, qk_norm_append_kernel<T><<<dim3((unsigned)N), 256, 0, (hipStream_t)stream>>>(
-                           (const T *)proj, ld, q_col, k_col, v_col, H * D, G * D, G * Dv, (const T *)wq, (const T *)wk, eps, (T *)q_out,
-                           (T *)k_cache, (T *)v_cache, slot));
+    if (rot_dims < 0 || rot_dims % 2 || rot_dims > D || (rot_dims && (!pos || !cos_t || !sin_t)) || (pairing != JL_ROT_HALVES && pairing != JL_ROT_NEIGHBOURS))
+        return jl_fail(JL_E_INVALID, "jl_qk_norm_append: a rotation needs an even width up to D, positions, angle tables and a known pairing");
+    hipStream_t st = (hipStream_t)stream;
+    const int HD = H * D, GD = G * D, GDv = G * Dv;
+    const uintptr_t al = dtype == JL_BF16 ? 8 : 16;
+    bool vec = D % 4 == 0 && GDv % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && v_col % 4 == 0 && rot_dims % 4 == 0 &&
+               (rot_dims == 0 || pairing == JL_ROT_NEIGHBOURS) && HD <= 8192 && GD <= 8192;
+    for (const void *ptr : {proj, wq, wk, (const void *)q_out, (const void *)k_cache, (const void *)v_cache}) vec = vec && (uintptr_t)ptr % al == 0;
+    if (vec) {
+#define QKV_CASE(Q, K) JL_DISPATCH(dtype, (qk_norm_append_vec_kernel<T, Q, K><<<dim3((unsigned)N), 256, 0, st>>>(                                  \
+                               (const T *)proj, ld, q_col, k_col, v_col, HD, GD, GDv, D, (const T *)wq, (const T *)wk, eps, (T *)q_out,            \
+                               (T *)k_cache, (T *)v_cache, slot, rot_dims, pos, cos_t, sin_t)))
+        if (HD <= 1024 && GD <= 1024) QKV_CASE(1, 1);
+        else if (HD <= 2048 && GD <= 1024) QKV_CASE(2, 1);
+        else if (HD <= 4096 && GD <= 1024) QKV_CASE(4, 1);
+        else QKV_CASE(8, 8);
+#undef QKV_CASE
+        return jl_check_launch("qk_norm_append_vec_kernel");
+    }
+    JL_DISPATCH(dtype, qk_norm_append_kernel<T><<<dim3((unsigned)N), 256, 0, st>>>(
+                           (const T *)proj, ld, q_col, k_col, v_col, HD, GD, GDv, D, (const T *)wq, (const T *)wk, eps, (T *)q_out,
+                           (T *)k_cache, (T *)v_cache, slot, rot_dims, pairing, pos, cos_t, sin_t));
     return jl_check_launch("qk_norm_append_kernel");
 }
 
@@ -104,7 +216,8 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_window_kernel(jl_attn_args a
     float *talk = sm + H * TQ;                          // [H][H]
     const int window = a.window > 0 ? a.window : 0x3fffffff;
     const int i_max = i0 + cnt - 1;
-    const int lo = i0 - window + 1 > 0 ? i0 - window + 1 : 0;
+    const int chunk = a.chunk;
+    const int lo = chunk > 0 ? i0 - i0 % chunk : (i0 - window + 1 > 0 ? i0 - window + 1 : 0);      // lowest key the tile's first row sees
     const int kf_end = a.keep_first < lo ? a.keep_first : lo;
     const int n_keys = kf_end + (i_max + 1 - lo);
     const int *bt = a.block_tables + (int64_t)b * a.bt_stride;
@@ -136,7 +249,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_window_kernel(jl_attn_args a
                 const int g = e / (cnt * nk), r = e - g * (cnt * nk), ii = r / nk, jj = r - ii * nk;
                 const int u = u0 + jj, j = u < kf_end ? u : lo + (u - kf_end), i = i0 + ii;
                 float s = -INFINITY;
-                if (j <= i && (i - j < window || j < a.keep_first)) {
+                if (j <= i && (chunk > 0 ? j >= i - i % chunk : (i - j < window || j < a.keep_first))) {
                     const float *qp = Qs + (ii * H + g) * D, *kp = KV + ((g / rep) * TK + jj) * kstride;
                     float dot = 0.f;
                     for (int d = 0; d < D; ++d) dot += qp[d] * kp[d];
@@ -145,6 +258,7 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_window_kernel(jl_attn_args a
                         const int n = i - j < a.lut_len ? i - j : a.lut_len - 1;
                         s += a.rel[(a.lut ? a.lut[n] : n) * H + g];
                     }
+                    if (a.softcap > 0.f) s = a.softcap * tanhf(s / a.softcap);
                 }
                 S[(g * TQ + ii) * TK + jj] = s;
             }
@@ -207,10 +321,10 @@ __global__ __launch_bounds__(ATT_THREADS) void attn_window_kernel(jl_attn_args a
         const int e = x * ATT_THREADS + tid;
         if (e < cnt * H * Dv) {
             const int ii = e / (H * Dv), r = e - ii * (H * Dv);
-            float v = acc[x];
+            float v = acc[x] * a.out_scale;
             if (gate) v *= 1.0f / (1.0f + expf(-ld_f(gate + (int64_t)(row0 + ii) * a.gate_ld + (a.gate_heads ? r / Dv : r))));
-            if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[(int64_t)(row0 + ii) * (H * Dv) + r] = v;
-            else st_f(out + (int64_t)(row0 + ii) * (H * Dv) + r, v);
+            if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[(int64_t)(row0 + ii) * a.out_ld + r] = v;
+            else st_f(out + (int64_t)(row0 + ii) * a.out_ld + r, v);
         }
     }
 }
@@ -318,7 +432,8 @@ __global__ __launch_bounds__(512) void attn_mfma_kernel(jl_attn_args a, int mode
     int *pageS = (int *)(biasS + H * 64);                          // [AM_PAGES] this request's page table up to the tile's last key
     const int window = a.window > 0 ? a.window : 0x3fffffff;
     const int i_max = i0 + cnt - 1;
-    const int lo = i0 - window + 1 > 0 ? i0 - window + 1 : 0;
+    const int chunk = a.chunk;
+    const int lo = chunk > 0 ? i0 - i0 % chunk : (i0 - window + 1 > 0 ? i0 - window + 1 : 0);      // lowest key the tile's first row sees
     const int kf_end = a.keep_first < lo ? a.keep_first : lo;
     const int n_keys = kf_end + (i_max + 1 - lo);
     const int *bt = a.block_tables + (int64_t)b * a.bt_stride;
@@ -441,7 +556,7 @@ __global__ __launch_bounds__(512) void attn_mfma_kernel(jl_attn_args a, int mode
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int ii = 8 * (r >> 2) + 4 * hi + (r & 3), i = i0 + ii;
-                    const bool ok = ii < cnt && l32 < nk && j <= i && (i - j < window || j < a.keep_first);
+                    const bool ok = ii < cnt && l32 < nk && j <= i && (chunk > 0 ? j >= i - i % chunk : (i - j < window || j < a.keep_first));
                     float s = -INFINITY;
                     if (ok) {
                         s = sc[r] * a.scale;
@@ -453,6 +568,7 @@ __global__ __launch_bounds__(512) void attn_mfma_kernel(jl_attn_args a, int mode
                                 s += a.rel[(a.lut ? a.lut[n] : n) * H + g];
                             }
                         }
+                        if (a.softcap > 0.f) s = soft_cap_fast(s, a.softcap);
                     }
                     if (sweep == 0) {
                         const float t = fmaxf(m_run[x][r], s);
@@ -582,10 +698,10 @@ __global__ __launch_bounds__(512) void attn_mfma_kernel(jl_attn_args a, int mode
                 const int ii = 8 * (r >> 2) + 4 * hi + (r & 3);
                 if (ii >= cnt) continue;
                 const int col = h * Dv + 32 * t + l32;
-                float v = acc[x][t][r];
+                float v = acc[x][t][r] * a.out_scale;
                 if (gate) v *= 1.0f / (1.0f + __expf(-ld_f(gate + (int64_t)(row0 + ii) * a.gate_ld + (a.gate_heads ? h : col))));
-                if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[(int64_t)(row0 + ii) * (H * Dv) + col] = v;
-                else st_f(out + (int64_t)(row0 + ii) * (H * Dv) + col, v);
+                if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[(int64_t)(row0 + ii) * a.out_ld + col] = v;
+                else st_f(out + (int64_t)(row0 + ii) * a.out_ld + col, v);
             }
         }
     }
@@ -609,17 +725,18 @@ __global__ __launch_bounds__(256) void attn_pack_q_kernel(const bf16_t *__restri
 // out = gate * the sum of the splits' shares, in split order
 __global__ __launch_bounds__(256) void attn_join_kernel(const float *__restrict__ po, int S, int64_t total, int width,
                                                          const bf16_t *__restrict__ gate, int64_t gate_ld, int gate_every,
-                                                         bf16_t *__restrict__ out, int out_f32) {
+                                                         bf16_t *__restrict__ out, int out_f32, int64_t out_ld, float out_scale) {
     const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (e >= total) return;
     float v = 0.f;
     for (int sp = 0; sp < S; ++sp) v += po[(int64_t)sp * total + e];
+    const int64_t row = e / width, o = row * out_ld + (e - row * width);
+    v *= out_scale;
     if (gate) {
-        const int64_t row = e / width;
         v *= 1.0f / (1.0f + __expf(-ld_f(gate + row * gate_ld + (e - row * width) / gate_every)));      // gate_every = Dv: one gate per head
     }
-    if (out_f32) ((float *)out)[e] = v;
-    else st_f(out + e, v);
+    if (out_f32) ((float *)out)[o] = v;
+    else st_f(out + o, v);
 }
 
 static bool am_fits(int dtype, int H, int G, int D, int Dv) {
@@ -647,7 +764,7 @@ template <int HPW, int NDV> static int am_launch(const jl_attn_args &a, hipStrea
     const int64_t total = (int64_t)a.n_rows * a.H * a.Dv;
     attn_join_kernel<<<dim3((unsigned)((total + 255) / 256)), 256, 0, st>>>(a.scratch + (int64_t)a.n_tiles * a.splits * a.H * AM_T * 2, a.splits, total,
                                                                           a.H * a.Dv, (const bf16_t *)a.gate, a.gate_ld, a.gate_heads ? a.Dv : 1, (bf16_t *)a.out,
-                                                                          a.out_dtype == JL_OUT_F32);
+                                                                          a.out_dtype == JL_OUT_F32, a.out_ld, a.out_scale);
     return jl_check_launch("attn_mfma_kernel (split keys)");
 }
 
@@ -676,6 +793,9 @@ extern "C" int jl_attn_window(const jl_attn_args *ap, void *stream) {
         return jl_fail(JL_E_INVALID, "jl_attn_window: value heads must divide the key heads, and row strides hold a row");
     if (a.out_dtype != JL_OUT_SAME && a.out_dtype != JL_OUT_F32) return jl_fail(JL_E_INVALID, "jl_attn_window: unknown out_dtype");
     if (a.dtype == JL_F32) a.out_dtype = JL_OUT_SAME;
+    if (a.out_ld <= 0) a.out_ld = (int64_t)a.H * a.Dv;
+    if (a.out_ld < (int64_t)a.H * a.Dv) return jl_fail(JL_E_INVALID, "jl_attn_window: the output rows do not fit their stride");
+    if (a.chunk > 0 && (a.window > 0 || a.keep_first > 0)) return jl_fail(JL_E_INVALID, "jl_attn_window: chunks exclude a window and kept first tokens");
     hipStream_t st = (hipStream_t)stream;
     if (a.splits > 1 && (!a.scratch || a.n_rows <= 0 || !(a.TQ == AM_T && am_fits(a.dtype, a.H, a.G, a.D, a.Dv) && am_strides_ok(a.k_ld, a.v_ld))))
         return jl_fail(JL_E_INVALID, "jl_attn_window: split keys need the matrix-core kernel, a scratch and the row count");

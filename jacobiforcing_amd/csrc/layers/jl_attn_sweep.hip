@@ -52,7 +52,8 @@ __global__ __launch_bounds__(AS_THREADS) void attn_sweep_kernel(jl_attn_args a, 
     float *lS = alphaS + AS_T;                                      // [32] final sums
     const int window = a.window > 0 ? a.window : 0x3fffffff;
     const int i_max = i0 + cnt - 1;
-    const int lo = i0 - window + 1 > 0 ? i0 - window + 1 : 0;
+    const int chunk = a.chunk;
+    const int lo = chunk > 0 ? i0 - i0 % chunk : (i0 - window + 1 > 0 ? i0 - window + 1 : 0);      // lowest key the tile's first row sees
     const int n_keys = i_max + 1 - lo;
     const int *bt = a.block_tables + (int64_t)b * a.bt_stride;
     const bf16_t *kc = (const bf16_t *)a.k_cache + (int64_t)c * D;
@@ -74,7 +75,7 @@ __global__ __launch_bounds__(AS_THREADS) void attn_sweep_kernel(jl_attn_args a, 
     }
     // the row this thread helps to reduce: row tid / 8, keys 4 * (tid % 8) .. + 3
     const int rr = tid >> 3, rc = (tid & 7) * 4;
-    const int r_i = i0 + rr / HF;
+    const int r_i = i0 + rr / HF, r_lo = chunk > 0 ? r_i - r_i % chunk : r_i - window + 1;      // the row's keys: r_lo .. r_i
     const bool r_ok = rr < TQ * HF && rr / HF < cnt && h0 + rr % HF < h_end;
     float m_run = -INFINITY, l_run = 0.f;
     // a sink acts like one extra score that attends to nothing: the row's statistics start from (sink, 1), in the first share of the keys only
@@ -150,8 +151,10 @@ __global__ __launch_bounds__(AS_THREADS) void attn_sweep_kernel(jl_attn_args a, 
             for (int x = 0; x < 4; ++x) {
                 const int jj = rc + x, j = lo + u0 + jj;
                 float v = Sp[rr * 33 + jj] + Sp[(AS_T + rr) * 33 + jj] + Sp[(2 * AS_T + rr) * 33 + jj] + Sp[(3 * AS_T + rr) * 33 + jj];
-                const bool ok = r_ok && jj < nk && j <= r_i && r_i - j < window;
-                s[x] = ok ? v * a.scale : -INFINITY;
+                const bool ok = r_ok && jj < nk && j <= r_i && j >= r_lo;
+                v *= a.scale;
+                if (a.softcap > 0.f) v = soft_cap_fast(v, a.softcap);
+                s[x] = ok ? v : -INFINITY;
                 mx = fmaxf(mx, s[x]);
             }
             mx = fmaxf(mx, __shfl_xor(mx, 1, 64));
@@ -226,8 +229,8 @@ __global__ __launch_bounds__(AS_THREADS) void attn_sweep_kernel(jl_attn_args a, 
         for (int t = 0; t < NT; ++t) {
             const int col = 32 * (AS_WAVES * t + wave) + l32;
             if (col - l32 >= Dv) continue;
-            const int64_t o = ((int64_t)(row0 + ii) * H + hh) * Dv + col;
-            float v = acc[t][r] * inv;
+            const int64_t o = (int64_t)(row0 + ii) * a.out_ld + hh * Dv + col;
+            float v = acc[t][r] * inv * a.out_scale;
             if (a.gate) v *= 1.0f / (1.0f + __expf(-ld_f((const bf16_t *)a.gate + (int64_t)(row0 + ii) * a.gate_ld + (a.gate_heads ? hh : hh * Dv + col))));
             if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[o] = v;
             else st_f(out + o, v);
@@ -264,7 +267,8 @@ __global__ __launch_bounds__(256) void attn_sweep_join_kernel(jl_attn_args a, in
         if (row >= TQ * HF || ii >= cnt || hh >= h_end) continue;
         float v = 0.f;
         for (int sp = 0; sp < S; ++sp) v += wS[row * 64 + sp] * base[sp * share + row * (Dv + 2) + col];
-        const int64_t o = ((int64_t)(row0 + ii) * H + hh) * Dv + col;
+        const int64_t o = (int64_t)(row0 + ii) * a.out_ld + hh * Dv + col;
+        v *= a.out_scale;
         if (a.gate) v *= 1.0f / (1.0f + __expf(-ld_f((const bf16_t *)a.gate + (int64_t)(row0 + ii) * a.gate_ld + (a.gate_heads ? hh : hh * Dv + col))));
         if (a.out_dtype == JL_OUT_F32) ((float *)a.out)[o] = v;
         else st_f(out + o, v);
@@ -312,7 +316,8 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
     int *pageS = (int *)(buf0 + 2 * buf_elems);
     const int window = a.window > 0 ? a.window : 0x3fffffff;
     const int i_max = i0 + cnt - 1;
-    const int lo = i0 - window + 1 > 0 ? i0 - window + 1 : 0;
+    const int chunk = a.chunk;
+    const int lo = chunk > 0 ? i0 - i0 % chunk : (i0 - window + 1 > 0 ? i0 - window + 1 : 0);      // lowest key the tile's first row sees
     const int n_keys = i_max + 1 - lo;
     const int *bt = a.block_tables + (int64_t)b * a.bt_stride;
     const bf16_t *kc = (const bf16_t *)a.k_cache + (int64_t)c * D;
@@ -329,7 +334,7 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
     // this lane's row: (query R / HF, head h0 + R % HF), R = 32 * wave + l32; both half-wavefronts hold it
     const int R = 32 * wave + l32, ii = R / HF, hh = h0 + R % HF;
     const bool ok = R < TQ * HF && ii < cnt && hh < h_end;
-    const int qi = i0 + ii;
+    const int qi = i0 + ii, q_lo = chunk > 0 ? qi - qi % chunk : qi - window + 1;                 // the row's keys: q_lo .. qi
     as_bf16x4 qf[QS];
     {
         const bf16_t *qp = (const bf16_t *)a.q + ((int64_t)(row0 + ii) * H + hh) * D + 4 * hi;
@@ -348,6 +353,8 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
         for (int r = 0; r < 16; ++r) acc[t][r] = 0.f;
     // the queries this wavefront's rows belong to (none: it only helps to load)
     const int wq_first = (32 * wave) / HF, wq_last = (32 * wave + 31) / HF < cnt - 1 ? (32 * wave + 31) / HF : cnt - 1;
+    const int wlo_first = chunk > 0 ? (i0 + wq_first) - (i0 + wq_first) % chunk : i0 + wq_first - window + 1;       // lowest keys of the first and the last of them
+    const int wlo_last = chunk > 0 ? (i0 + wq_last) - (i0 + wq_last) % chunk : i0 + wq_last - window + 1;
     const bool wave_live = 32 * wave < TQ * HF && wq_first < cnt;
     const bool wave_full = 32 * wave + 31 < TQ * HF && (32 * wave + 31) / HF < cnt && h0 + HF <= h_end;     // all 32 rows are rows of the tile
 
@@ -428,7 +435,7 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
         const bf16_t *Ks = buf0 + tsel * buf_elems, *Vs = v_in_k ? Ks : Ks + AS_T * KROW;
         const int j0 = lo + u0;                                     // position of the tile's first key
         // wavefront-uniform: keys all behind its last query, or all before its first query's window
-        if (wave_live && j0 <= i0 + wq_last && j0 + nk - 1 >= i0 + wq_first - window + 1) {
+        if (wave_live && j0 <= i0 + wq_last && j0 + nk - 1 >= wlo_first) {
         as_f32x16 sc;
 #pragma unroll
         for (int r = 0; r < 16; ++r) sc[r] = 0.f;
@@ -440,16 +447,22 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
         }
         float mx = -INFINITY;
         // wavefront-uniform: a full tile whose keys every row of the wavefront sees needs no mask
-        const bool inside = nk == AS_T && wave_full && j0 + AS_T - 1 <= i0 + wq_first && i0 + wq_last - j0 < window;
+        const bool inside = nk == AS_T && wave_full && j0 + AS_T - 1 <= i0 + wq_first && j0 >= wlo_last;
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sc[r] *= a.scale;
+        if (a.softcap > 0.f) {
+#pragma unroll
+            for (int r = 0; r < 16; ++r) sc[r] = soft_cap_fast(sc[r], a.softcap);
+        }
         if (inside) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r) { sc[r] *= a.scale; mx = fmaxf(mx, sc[r]); }
+            for (int r = 0; r < 16; ++r) mx = fmaxf(mx, sc[r]);
         } else {
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int kk = 8 * (r >> 2) + 4 * hi + (r & 3), j = j0 + kk;
-                const bool vis = ok && kk < nk && j <= qi && qi - j < window;
-                sc[r] = vis ? sc[r] * a.scale : -INFINITY;
+                const bool vis = ok && kk < nk && j <= qi && j >= q_lo;
+                sc[r] = vis ? sc[r] : -INFINITY;
                 mx = fmaxf(mx, sc[r]);
             }
         }
@@ -493,7 +506,8 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
     const bf16_t *gate = (const bf16_t *)a.gate;
     float gh = 1.0f;
     if (gate && a.gate_heads) gh = 1.0f / (1.0f + __expf(-ld_f(gate + (int64_t)(row0 + ii) * a.gate_ld + hh)));
-    const int64_t obase = ((int64_t)(row0 + ii) * H + hh) * Dv;
+    const int64_t obase = (int64_t)(row0 + ii) * a.out_ld + hh * Dv;
+    gh *= a.out_scale;
 #pragma unroll
     for (int t = 0; t < NDV; ++t) {
         if (32 * t >= Dv) continue;
@@ -570,6 +584,9 @@ extern "C" int jl_attn_sweep(const jl_attn_args *ap, void *stream) {
         return jl_fail(JL_E_INVALID, "jl_attn_sweep: bfloat16, key width a multiple of 8 up to %d, value width a multiple of 32 up to 512, row strides in "
                        "multiples of 4; values inside the key rows need one key head", 8 * AS_WAVES * AS_QSTEPS);
     if (a.out_dtype != JL_OUT_SAME && a.out_dtype != JL_OUT_F32) return jl_fail(JL_E_INVALID, "jl_attn_sweep: unknown out_dtype");
+    if (a.out_ld <= 0) a.out_ld = (int64_t)a.H * a.Dv;
+    if (a.out_ld < (int64_t)a.H * a.Dv || a.out_ld % 4) return jl_fail(JL_E_INVALID, "jl_attn_sweep: the output's row stride holds a row and is a multiple of four");
+    if (a.chunk > 0 && a.window > 0) return jl_fail(JL_E_INVALID, "jl_attn_sweep: chunks exclude a window");
     const int hf = as_heads_per_tile(a.H, a.G), hb = as_head_blocks(a.H, a.G), tq = AS_T / hf;
     if (a.TQ == AR_ROWS / hf && a.TQ != tq) {                       // tiles of up to 128 rows: every wavefront keeps its rows to itself
         if (a.splits > 1 || !ar_fits(a.dtype, a.H, a.G, a.Gv, a.D, a.Dv, a.k_ld, a.v_ld, v_in_k))

@@ -32,6 +32,20 @@ __device__ __forceinline__ float ld_any(const void *p, int dtype, int64_t i) {
     return dtype == JL_BF16 ? ld_f((const bf16_t *)p + i) : ((const float *)p)[i];
 }
 
+// four elements at a time (8 bytes of bfloat16, 16 of float, aligned to that)
+__device__ __forceinline__ void ld4_f(const float *p, float (&v)[4]) { const float4 t = *(const float4 *)p; v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w; }
+__device__ __forceinline__ void ld4_f(const bf16_t *p, float (&v)[4]) {
+    const uint2 t = *(const uint2 *)p;
+    v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u); v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
+}
+__device__ __forceinline__ void st4_f(float *p, const float (&v)[4]) { *(float4 *)p = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void st4_f(bf16_t *p, const float (&v)[4]) {
+    bf16_t h[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) st_f(h + i, v[i]);
+    *(uint2 *)p = make_uint2((uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16));
+}
+
 __device__ __forceinline__ float wave_sum_f32(float v) {
 #pragma unroll
     for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off, 64);
@@ -49,6 +63,12 @@ __device__ __forceinline__ float block_sum_f32(float v, float *red) {
     for (int i = 0; i < nw; ++i) s += red[i];
     return s;
 }
+
+// cap * tanh(s / cap) with tanh(z) = 1 - 2 / (1 + exp(2 z)): a few 1e-7 of cap off, for scores that bfloat16 operands made
+__device__ __forceinline__ float soft_cap_fast(float s, float cap) {
+    return cap - 2.0f * cap * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * s * __builtin_amdgcn_rcpf(cap)));
+}
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // gated units of a feed-forward (jl_gated_act, and the grouped product that applies them in its epilogue)
 // 0.5 z (1 + tanh(u)) = z sigmoid(2u), u = sqrt(2/pi) (z + 0.044715 z^3)

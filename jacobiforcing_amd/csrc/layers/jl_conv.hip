@@ -139,20 +139,33 @@ extern "C" int jl_causal_conv_carry(const float *x, const int32_t *seq, int32_t 
     return jl_check_launch("causal_conv_carry_kernel");
 }
 
-// ---- short causal convolution of a column range of a projection, with an activation, no residual ---------------------------------------------
-//   out[t, c] = act(sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start; float out)
-// A workgroup walks CONV_ROWS consecutive rows, a thread owns a channel and keeps the last taps - 1 inputs in registers.  The tail
-// (float [slots, taps - 1, C]) is read for the inputs before the step and moved on here by requests with ONE row; requests with more rows
-// leave that to short_conv_carry_kernel, enqueued after every row has read.
-template <typename T, int TAPS>
-__global__ __launch_bounds__(256) void short_conv_kernel(const T *__restrict__ x, int64_t ld, int col, const T *__restrict__ w, const int32_t *__restrict__ row_req,
-                                                          const int32_t *__restrict__ seq, float *tail, int64_t N, int C, int act, float *__restrict__ out) {
+// ---- short causal convolution of a column range of a projection, with an optional bias and an activation, no residual -----------------------
+//   out[t, c] = act(bias[c] + sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start)
+// A workgroup walks CONV_ROWS consecutive rows, a thread owns VC channels (one, or four with 8- or 16-byte loads) and keeps the last taps - 1
+// inputs in registers.  The tail (float [slots, taps - 1, C]) is read for the inputs before the step and moved on here by requests with
+// ONE row; requests with more rows leave that to short_conv_carry_kernel, enqueued after every row has read.
+template <int VC, typename P> __device__ __forceinline__ void conv_ld(const P *p, float (&v)[VC]) {
+    if constexpr (VC == 4) ld4_f(p, v);
+    else v[0] = ld_f(p);
+}
+template <int VC, typename P> __device__ __forceinline__ void conv_st(P *p, const float (&v)[VC]) {
+    if constexpr (VC == 4) st4_f(p, v);
+    else st_f(p, v[0]);
+}
+template <typename T, typename TO, int TAPS, int VC>
+__global__ __launch_bounds__(256) void short_conv_kernel(const T *__restrict__ x, int64_t ld, int col, const T *__restrict__ w, const T *__restrict__ bias,
+                                                          const int32_t *__restrict__ row_req, const int32_t *__restrict__ seq, float *tail, int64_t N, int C, int act,
+                                                          TO *__restrict__ out) {
     constexpr int KEEP = TAPS - 1;
-    const int c = blockIdx.y * 256 + threadIdx.x;
+    const int c = (blockIdx.y * 256 + threadIdx.x) * VC;
     if (c >= C) return;
-    float wv[TAPS], win[KEEP > 0 ? KEEP : 1];
+    float wv[TAPS][VC], win[KEEP > 0 ? KEEP : 1][VC], bv[VC];
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) wv[j] = ld_f(w + (int64_t)c * TAPS + j);
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < VC; ++e) wv[j][e] = ld_f(w + (int64_t)(c + e) * TAPS + j);
+#pragma unroll
+    for (int e = 0; e < VC; ++e) bv[e] = bias ? ld_f(bias + c + e) : 0.f;
     int prev_req = -1;
     const int64_t n0 = (int64_t)blockIdx.x * CONV_ROWS;
     for (int r = 0; r < CONV_ROWS && n0 + r < N; ++r) {
@@ -165,24 +178,30 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T *__restrict__ x
 #pragma unroll
             for (int s2 = 0; s2 < KEEP; ++s2) {
                 const int u = t - KEEP + s2;
-                float v = 0.f;
-                if (u >= 0) v = ld_f(x + (int64_t)(row0 + u) * ld + col + c);
-                else if (pos0 + u >= 0) v = tail[((int64_t)slot * KEEP + (KEEP + u)) * C + c];
-                win[s2] = v;
+#pragma unroll
+                for (int e = 0; e < VC; ++e) win[s2][e] = 0.f;
+                if (u >= 0) conv_ld<VC>(x + (int64_t)(row0 + u) * ld + col + c, win[s2]);
+                else if (pos0 + u >= 0) conv_ld<VC>(tail + ((int64_t)slot * KEEP + (KEEP + u)) * C + c, win[s2]);
             }
             prev_req = req;
         }
-        const float cur = ld_f(x + n * ld + col + c);
-        float a = wv[KEEP] * cur;
+        float cur[VC], a[VC];
+        conv_ld<VC>(x + n * ld + col + c, cur);
 #pragma unroll
-        for (int s2 = 0; s2 < KEEP; ++s2) a += wv[s2] * win[s2];
-        out[n * C + c] = act == JL_ACT_SILU ? silu_f(a) : a;
+        for (int e = 0; e < VC; ++e) {
+            a[e] = bv[e] + wv[KEEP][e] * cur[e];
 #pragma unroll
-        for (int s2 = 0; s2 + 1 < KEEP; ++s2) win[s2] = win[s2 + 1];
-        if (KEEP > 0) win[KEEP - 1] = cur;
+            for (int s2 = 0; s2 < KEEP; ++s2) a[e] += wv[s2][e] * win[s2][e];
+            if (act == JL_ACT_SILU) a[e] = silu_f(a[e]);
+        }
+        conv_st<VC>(out + n * C + c, a);
+#pragma unroll
+        for (int s2 = 0; s2 < KEEP; ++s2)
+#pragma unroll
+            for (int e = 0; e < VC; ++e) win[s2][e] = s2 + 1 < KEEP ? win[s2 + 1 < KEEP ? s2 + 1 : s2][e] : cur[e];
         if (count == 1 && KEEP > 0) {
 #pragma unroll
-            for (int s2 = 0; s2 < KEEP; ++s2) tail[((int64_t)slot * KEEP + s2) * C + c] = win[s2];
+            for (int s2 = 0; s2 < KEEP; ++s2) conv_st<VC>(tail + ((int64_t)slot * KEEP + s2) * C + c, win[s2]);
         }
     }
 }
@@ -209,23 +228,37 @@ __global__ __launch_bounds__(256) void short_conv_carry_kernel(const T *__restri
         if (s < keep) tail[((int64_t)slot * keep + s) * C + c] = v[s];
 }
 
-template <typename T, int TAPS>
-static void short_conv_launch(const void *x, int64_t ld, int col, const void *w, const int32_t *row_req, const int32_t *seq, float *tail, int64_t N, int C,
-                              int act, float *out, hipStream_t st) {
-    const dim3 grid((unsigned)((N + CONV_ROWS - 1) / CONV_ROWS), (unsigned)((C + 255) / 256));
-    short_conv_kernel<T, TAPS><<<grid, 256, 0, st>>>((const T *)x, ld, col, (const T *)w, row_req, seq, tail, N, C, act, out);
+template <typename T, typename TO, int TAPS>
+static void short_conv_launch(const void *x, int64_t ld, int col, const void *w, const void *bias, const int32_t *row_req, const int32_t *seq, float *tail, int64_t N,
+                              int C, int act, void *out, hipStream_t st) {
+    const unsigned gx = (unsigned)((N + CONV_ROWS - 1) / CONV_ROWS);
+    auto al = [](const void *q, uintptr_t a) { return ((uintptr_t)q % a) == 0; };
+    if (C % 4 == 0 && col % 4 == 0 && ld % 4 == 0 && al(x, 4 * sizeof(T)) && al(out, 4 * sizeof(TO)) && al(tail, 16))
+        short_conv_kernel<T, TO, TAPS, 4><<<dim3(gx, (unsigned)((C / 4 + 255) / 256)), 256, 0, st>>>((const T *)x, ld, col, (const T *)w, (const T *)bias, row_req, seq,
+                                                                                                     tail, N, C, act, (TO *)out);
+    else
+        short_conv_kernel<T, TO, TAPS, 1><<<dim3(gx, (unsigned)((C + 255) / 256)), 256, 0, st>>>((const T *)x, ld, col, (const T *)w, (const T *)bias, row_req, seq, tail,
+                                                                                                 N, C, act, (TO *)out);
 }
 
-extern "C" int jl_short_conv(const void *x, int dtype, int64_t ld, int32_t col, const void *w, const int32_t *row_req, const int32_t *seq, int32_t B,
-                             int32_t max_count, float *tail, int64_t N, int32_t C, int32_t taps, int32_t act, float *out, void *stream) {
+extern "C" int jl_short_conv(const void *x, int dtype, int64_t ld, int32_t col, const void *w, const void *bias, const int32_t *row_req, const int32_t *seq, int32_t B,
+                             int32_t max_count, float *tail, int64_t N, int32_t C, int32_t taps, int32_t act, void *out, int out_dtype, void *stream) {
     if (N <= 0) return JL_OK;
     if (!x || !w || !row_req || !seq || !out || C <= 0 || col < 0 || col + (int64_t)C > ld || taps < 1 || taps > 8 || (taps > 1 && !tail))
         return jl_fail(JL_E_INVALID, "jl_short_conv: null pointer, columns outside the row, or taps outside 1..8");
     if (act != JL_ACT_SILU && act != JL_ACT_NONE) return jl_fail(JL_E_INVALID, "jl_short_conv: unknown activation %d", act);
+    if (out_dtype != JL_F32 && out_dtype != dtype) return jl_fail(JL_E_INVALID, "jl_short_conv: the output is float or of the input's dtype");
     hipStream_t st = (hipStream_t)stream;
-#define CONV_CASE(TP) case TP: JL_DISPATCH(dtype, (short_conv_launch<T, TP>(x, ld, col, w, row_req, seq, tail, N, C, act, out, st))); break
+#define CONV_ARGS x, ld, col, w, bias, row_req, seq, tail, N, C, act, out, st
+#define CONV_CASE(TP)                                                                                       \
+    case TP:                                                                                                \
+        if (dtype != JL_BF16) short_conv_launch<float, float, TP>(CONV_ARGS);                               \
+        else if (out_dtype == JL_BF16) short_conv_launch<bf16_t, bf16_t, TP>(CONV_ARGS);                    \
+        else short_conv_launch<bf16_t, float, TP>(CONV_ARGS);                                               \
+        break
     switch (taps) { CONV_CASE(1); CONV_CASE(2); CONV_CASE(3); CONV_CASE(4); CONV_CASE(5); CONV_CASE(6); CONV_CASE(7); CONV_CASE(8); }
 #undef CONV_CASE
+#undef CONV_ARGS
     int rc = jl_check_launch("short_conv_kernel");
     if (rc != JL_OK || taps == 1 || max_count <= 1) return rc;
     JL_DISPATCH(dtype, short_conv_carry_kernel<T><<<dim3((unsigned)((C + 255) / 256), (unsigned)B), 256, 0, st>>>((const T *)x, ld, col, seq, tail, C, taps));

@@ -11,8 +11,6 @@
 // thread per token evaluates the decay and the step size; the per-head sums of squares of the outputs are reduced once per group.
 constexpr int DL_TT = 8;
 
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
 template <typename T, typename TQ, int DMAX, int LPC>
 __global__ __launch_bounds__(1024) void delta_rule_kernel(const TQ *__restrict__ qkv, int64_t qkv_ld, int q_col, int k_col, int v_col,
                                                            const T *__restrict__ proj, int64_t ld, int a_col, int b_col, int g_col,

@@ -48,20 +48,6 @@ __global__ __launch_bounds__(256) void head_norm_append_kernel(const T *__restri
         for (int c = threadIdx.x; c < GDv; c += 256) v_cache[sl * GDv + c] = row[v_col + c];
 }
 
-// four elements at a time (8 bytes of bfloat16, 16 of float)
-__device__ __forceinline__ void ld4(const float *p, float (&v)[4]) { const float4 t = *(const float4 *)p; v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w; }
-__device__ __forceinline__ void ld4(const bf16_t *p, float (&v)[4]) {
-    const uint2 t = *(const uint2 *)p;
-    v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u); v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
-}
-__device__ __forceinline__ void st4(float *p, const float (&v)[4]) { *(float4 *)p = make_float4(v[0], v[1], v[2], v[3]); }
-__device__ __forceinline__ void st4(bf16_t *p, const float (&v)[4]) {
-    bf16_t h[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) st_f(h + i, v[i]);
-    *(uint2 *)p = make_uint2((uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16));
-}
-
 // The same with LPV lanes per D-vector (a power of two, 4 * LPV >= D, D % 4 == 0, every column offset and row stride a multiple of
 // four): a wavefront normalises 64 / LPV vectors at a time, four elements per lane and load.
 template <typename T>
@@ -84,8 +70,8 @@ __global__ __launch_bounds__(256) void head_norm_append_vec_kernel(const T *__re
     float cs[4] = {1.f, 1.f, 1.f, 1.f}, sn[4] = {0.f, 0.f, 0.f, 0.f};
     if (turn) {
         const int64_t a0 = (int64_t)pos[n] * half + (d < half ? d : d - half);
-        ld4(cos_t + a0, cs);
-        ld4(sin_t + a0, sn);
+        ld4_f(cos_t + a0, cs);
+        ld4_f(sin_t + a0, sn);
         if (d < half)                                           // first of a pair: u cos - v sin; second: v cos + u sin
 #pragma unroll
             for (int i = 0; i < 4; ++i) sn[i] = -sn[i];
@@ -97,10 +83,10 @@ __global__ __launch_bounds__(256) void head_norm_append_vec_kernel(const T *__re
         const int idx = is_q ? vec : vec - nq;
         const int head = idx / M, map = idx - head * M;
         float x[4] = {0.f, 0.f, 0.f, 0.f};
-        if (live) ld4(row + (is_q ? q_col : k_col) + (int64_t)idx * D + d, x);
+        if (live) ld4_f(row + (is_q ? q_col : k_col) + (int64_t)idx * D + d, x);
         if (live && turn) {
             float p[4];
-            ld4(row + (is_q ? q_col : k_col) + (int64_t)idx * D + pd, p);
+            ld4_f(row + (is_q ? q_col : k_col) + (int64_t)idx * D + pd, p);
 #pragma unroll
             for (int i = 0; i < 4; ++i) x[i] = x[i] * cs[i] + p[i] * sn[i];
         }
@@ -109,15 +95,15 @@ __global__ __launch_bounds__(256) void head_norm_append_vec_kernel(const T *__re
         if (!live) continue;
         const float r = 1.0f / sqrtf(ss / (float)D + eps) * (is_q ? temp : 1.0f);
         float g[4] = {1.f, 1.f, 1.f, 1.f};
-        if (is_q ? wq != nullptr : wk != nullptr) ld4((is_q ? wq : wk) + d, g);
+        if (is_q ? wq != nullptr : wk != nullptr) ld4_f((is_q ? wq : wk) + d, g);
 #pragma unroll
         for (int i = 0; i < 4; ++i) x[i] = x[i] * r * g[i];
         if (is_q) {
             T *dst = q_map_stride ? q_out + map * q_map_stride + n * ((int64_t)H * D) + (int64_t)head * D
                                   : q_out + n * ((int64_t)nq * D) + ((int64_t)map * H + head) * D;
-            st4(dst + d, x);
+            st4_f(dst + d, x);
         } else if (sl >= 0) {
-            st4(k_cache + sl * ((int64_t)nk * D) + ((int64_t)map * G + head) * D + d, x);
+            st4_f(k_cache + sl * ((int64_t)nk * D) + ((int64_t)map * G + head) * D + d, x);
         }
     }
     if (sl >= 0)

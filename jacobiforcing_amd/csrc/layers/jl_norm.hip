@@ -303,20 +303,8 @@ __global__ __launch_bounds__(256) void depth_mix_norm_kernel(const float *__rest
 // The same for widths in multiples of four with 16-byte aligned rows: a thread owns four consecutive channels per pass (16-byte loads and
 // stores of floats, 8-byte ones of bfloat16).  SHIFT: the token shift of single-row steps rides along.
 __device__ __forceinline__ void ld4_any(const void *p, int dtype, int64_t i, float (&v)[4]) {
-    if (dtype == JL_BF16) {
-        const uint2 t = *(const uint2 *)((const bf16_t *)p + i);
-        v[0] = __uint_as_float(t.x << 16); v[1] = __uint_as_float(t.x & 0xffff0000u); v[2] = __uint_as_float(t.y << 16); v[3] = __uint_as_float(t.y & 0xffff0000u);
-    } else {
-        const float4 t = *(const float4 *)((const float *)p + i);
-        v[0] = t.x; v[1] = t.y; v[2] = t.z; v[3] = t.w;
-    }
-}
-__device__ __forceinline__ void st4_f(float *p, const float (&v)[4]) { *(float4 *)p = make_float4(v[0], v[1], v[2], v[3]); }
-__device__ __forceinline__ void st4_f(bf16_t *p, const float (&v)[4]) {
-    bf16_t h[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) st_f(&h[i], v[i]);
-    *(uint2 *)p = make_uint2((uint32_t)h[0] | ((uint32_t)h[1] << 16), (uint32_t)h[2] | ((uint32_t)h[3] << 16));
+    if (dtype == JL_BF16) ld4_f((const bf16_t *)p + i, v);
+    else ld4_f((const float *)p + i, v);
 }
 
 template <typename T, bool SHIFT>
@@ -473,4 +461,212 @@ extern "C" int jl_softcap(float *z, int64_t total, float cap, void *stream) {
     if (!z || !(cap > 0.f)) return jl_fail(JL_E_INVALID, "jl_softcap: null pointer or a cap that is not positive");
     softcap_kernel<<<dim3((unsigned)((total + 255) / 256)), 256, 0, (hipStream_t)stream>>>(z, total, cap);
     return jl_check_launch("softcap_kernel");
+}
+
+// ---- sublayer output norm, residual update, next sublayer's norm: one workgroup per row -----------------------------------------------------
+//   x = x_in + rms_norm(y) * w_post + add_row;   out = rms_norm(x) * w_next, or x itself (plain)
+// A thread keeps its VI x 4 channels in registers from the first load to the last store.
+template <typename T, typename TY, int VI>
+__global__ __launch_bounds__(256) void sandwich_norm_vec_kernel(const float *x_in, float *x_out, const TY *__restrict__ y,
+                                                                 const float *__restrict__ w_post, const float *__restrict__ add_row, float eps,
+                                                                 const float *__restrict__ w_next, T *__restrict__ out, int64_t out_ld, int plain, int W) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int step = blockDim.x * 4;
+    float x[VI][4];
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c < W) ld4_f(x_in + n * W + c, x[i]);
+    }
+    if (y) {
+        float v[VI][4], ss = 0.f;
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int c = i * step + threadIdx.x * 4;
+            if (c < W) {
+                ld4_f(y + n * W + c, v[i]);
+                ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+            }
+        }
+        ss = block_sum_f32(ss, red);
+        const float r = 1.0f / sqrtf(ss / (float)W + eps);
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int c = i * step + threadIdx.x * 4;
+            if (c < W) {
+                float g[4];
+                ld4_f(w_post + c, g);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[i][e] += v[i][e] * r * g[e];
+            }
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c < W) {
+            if (add_row) {
+                float g[4];
+                ld4_f(add_row + c, g);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x[i][e] += g[e];
+            }
+            if (y || add_row) st4_f(x_out + n * W + c, x[i]);
+            ss += x[i][0] * x[i][0] + x[i][1] * x[i][1] + x[i][2] * x[i][2] + x[i][3] * x[i][3];
+        }
+    }
+    if (!out) return;
+    float r = 1.0f;
+    if (!plain) {
+        ss = block_sum_f32(ss, red);
+        r = 1.0f / sqrtf(ss / (float)W + eps);
+    }
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c < W) {
+            float g[4] = {1.f, 1.f, 1.f, 1.f};
+            if (!plain) ld4_f(w_next + c, g);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) g[e] *= x[i][e] * r;
+            st4_f(out + n * out_ld + c, g);
+        }
+    }
+}
+
+template <typename T, typename TY>
+__global__ __launch_bounds__(256) void sandwich_norm_kernel(const float *x_in, float *x_out, const TY *__restrict__ y, const float *__restrict__ w_post,
+                                                             const float *__restrict__ add_row, float eps, const float *__restrict__ w_next,
+                                                             T *__restrict__ out, int64_t out_ld, int plain, int W) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    float r = 0.f, ss = 0.f;
+    if (y) {
+        for (int c = threadIdx.x; c < W; c += 256) { const float v = ld_f(y + n * W + c); ss += v * v; }
+        r = 1.0f / sqrtf(block_sum_f32(ss, red) / (float)W + eps);
+    }
+    ss = 0.f;
+    for (int c = threadIdx.x; c < W; c += 256) {
+        float v = x_in[n * W + c];
+        if (y) v += ld_f(y + n * W + c) * r * w_post[c];
+        if (add_row) v += add_row[c];
+        if (y || add_row) x_out[n * W + c] = v;
+        ss += v * v;
+    }
+    if (!out) return;
+    const float rn = plain ? 1.0f : 1.0f / sqrtf(block_sum_f32(ss, red) / (float)W + eps);
+    const float *xr = (y || add_row) ? x_out : x_in;
+    for (int c = threadIdx.x; c < W; c += 256) st_f(out + n * out_ld + c, xr[n * W + c] * rn * (plain ? 1.0f : w_next[c]));
+}
+
+extern "C" int jl_sandwich_norm(const float *x_in, float *x_out, const void *y, int y_dtype, const float *w_post, const float *add_row, float eps,
+                                const float *w_next, void *out, int dtype, int64_t out_ld, int32_t plain, int64_t N, int32_t W, void *stream) {
+    if (N <= 0) return JL_OK;
+    if (!x_in || W <= 0 || (y && !w_post) || ((y || add_row) && !x_out) || (out && !plain && !w_next))
+        return jl_fail(JL_E_INVALID, "jl_sandwich_norm: null pointer or bad width");
+    if (out_ld <= 0) out_ld = W;
+    if (out_ld < W) return jl_fail(JL_E_INVALID, "jl_sandwich_norm: the output rows do not fit their stride");
+    hipStream_t st = (hipStream_t)stream;
+    auto al = [](const void *q, uintptr_t a) { return ((uintptr_t)q % a) == 0; };
+    const bool vec = W % 4 == 0 && W <= 8192 && out_ld % 4 == 0 && al(x_in, 16) && al(x_out, 16) && al(w_post, 16) && al(add_row, 16) && al(w_next, 16) &&
+                     al(y, y_dtype == JL_BF16 ? 8 : 16) && al(out, dtype == JL_BF16 ? 8 : 16);
+    const int threads = W >= 1024 ? 256 : (W / 4 + 63) / 64 * 64;
+#define SN_ARGS(TY) x_in, x_out, (const TY *)y, w_post, add_row, eps, w_next, (T *)out, out_ld, plain, W
+#define SN_CASE(TY)                                                                                                                       \
+    do {                                                                                                                                  \
+        if (!vec) JL_DISPATCH(dtype, (sandwich_norm_kernel<T, TY><<<dim3((unsigned)N), 256, 0, st>>>(SN_ARGS(TY))));                      \
+        else if (W <= 1024) JL_DISPATCH(dtype, (sandwich_norm_vec_kernel<T, TY, 1><<<dim3((unsigned)N), threads, 0, st>>>(SN_ARGS(TY)))); \
+        else if (W <= 2048) JL_DISPATCH(dtype, (sandwich_norm_vec_kernel<T, TY, 2><<<dim3((unsigned)N), threads, 0, st>>>(SN_ARGS(TY)))); \
+        else if (W <= 4096) JL_DISPATCH(dtype, (sandwich_norm_vec_kernel<T, TY, 4><<<dim3((unsigned)N), threads, 0, st>>>(SN_ARGS(TY)))); \
+        else JL_DISPATCH(dtype, (sandwich_norm_vec_kernel<T, TY, 8><<<dim3((unsigned)N), threads, 0, st>>>(SN_ARGS(TY))));                \
+    } while (0)
+    if (y_dtype == JL_BF16) SN_CASE(bf16_t);
+    else SN_CASE(float);
+#undef SN_CASE
+#undef SN_ARGS
+    return jl_check_launch("sandwich_norm_kernel");
+}
+
+// ---- norm over equal parts of a mixer's output with its gate: one workgroup per (row, part) -------------------------------------------------
+//   gate first:  v = raw * act(gate);  out = v / rms(v) * w * scale          gate last:  out = raw / rms(raw) * w * act(gate) * scale
+__device__ __forceinline__ float gate_act_f(float g, int act) {
+    const float s = 1.0f / (1.0f + expf(-g));
+    return act == JL_ACT_SILU ? g * s : s;
+}
+template <typename T, int VI>
+__global__ __launch_bounds__(256) void gated_norm_vec_kernel(const float *__restrict__ raw, const T *__restrict__ gate, int64_t gate_ld, const float *__restrict__ w,
+                                                              float eps, int act, int gate_first, float scale, T *__restrict__ out, int64_t out_ld, int C, int part) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int c0 = blockIdx.y * part, step = blockDim.x * 4;
+    float v[VI][4], g[VI][4], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c < part) {
+            ld4_f(raw + n * C + c0 + c, v[i]);
+            ld4_f(gate + n * gate_ld + c0 + c, g[i]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                g[i][e] = gate_act_f(g[i][e], act);
+                if (gate_first) v[i][e] *= g[i][e];
+                ss += v[i][e] * v[i][e];
+            }
+        }
+    }
+    ss = block_sum_f32(ss, red);
+    const float r = scale / sqrtf(ss / (float)part + eps);
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c < part) {
+            float wv[4];
+            ld4_f(w + c0 + c, wv);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) wv[e] *= v[i][e] * r * (gate_first ? 1.0f : g[i][e]);
+            st4_f(out + n * out_ld + c0 + c, wv);
+        }
+    }
+}
+template <typename T>
+__global__ __launch_bounds__(256) void gated_norm_kernel(const float *__restrict__ raw, const T *__restrict__ gate, int64_t gate_ld, const float *__restrict__ w,
+                                                          float eps, int act, int gate_first, float scale, T *__restrict__ out, int64_t out_ld, int C, int part) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int c0 = blockIdx.y * part;
+    float ss = 0.f;
+    for (int c = c0 + threadIdx.x; c < c0 + part; c += blockDim.x) {
+        float v = raw[n * C + c];
+        if (gate_first) v *= gate_act_f(ld_f(gate + n * gate_ld + c), act);
+        ss += v * v;
+    }
+    ss = block_sum_f32(ss, red);
+    const float r = scale / sqrtf(ss / (float)part + eps);
+    for (int c = c0 + threadIdx.x; c < c0 + part; c += blockDim.x)
+        st_f(out + n * out_ld + c, raw[n * C + c] * r * w[c] * gate_act_f(ld_f(gate + n * gate_ld + c), act));
+}
+
+extern "C" int jl_gated_norm(const float *raw, const void *gate, int dtype, int64_t gate_ld, const float *w, float eps, int32_t act, int32_t gate_first,
+                             float scale, void *out, int64_t out_ld, int64_t N, int32_t C, int32_t parts, void *stream) {
+    if (N <= 0) return JL_OK;
+    if (!raw || !gate || !w || !out || C <= 0 || parts <= 0 || C % parts || gate_ld < C || out_ld < C)
+        return jl_fail(JL_E_INVALID, "jl_gated_norm: null pointer, parts that do not divide the width, or rows that do not fit their stride");
+    if (act != JL_ACT_SILU && act != JL_ACT_SIGMOID) return jl_fail(JL_E_INVALID, "jl_gated_norm: unknown activation %d", act);
+    hipStream_t st = (hipStream_t)stream;
+    const int part = C / parts;
+    auto al = [](const void *q, uintptr_t a) { return ((uintptr_t)q % a) == 0; };
+    const uintptr_t ta = dtype == JL_BF16 ? 8 : 16;
+    const bool vec = part % 4 == 0 && part <= 8192 && gate_ld % 4 == 0 && out_ld % 4 == 0 && al(raw, 16) && al(w, 16) && al(gate, ta) && al(out, ta);
+    const dim3 grid((unsigned)N, (unsigned)parts);
+    const int per = vec ? part / 4 : part, threads = per >= 256 ? 256 : (per + 63) / 64 * 64;
+#define GN_ARGS raw, (const T *)gate, gate_ld, w, eps, act, gate_first, scale, (T *)out, out_ld, C, part
+    if (!vec) JL_DISPATCH(dtype, (gated_norm_kernel<T><<<grid, threads, 0, st>>>(GN_ARGS)));
+    else if (part <= 1024) JL_DISPATCH(dtype, (gated_norm_vec_kernel<T, 1><<<grid, threads, 0, st>>>(GN_ARGS)));
+    else if (part <= 2048) JL_DISPATCH(dtype, (gated_norm_vec_kernel<T, 2><<<grid, threads, 0, st>>>(GN_ARGS)));
+    else if (part <= 4096) JL_DISPATCH(dtype, (gated_norm_vec_kernel<T, 4><<<grid, threads, 0, st>>>(GN_ARGS)));
+    else JL_DISPATCH(dtype, (gated_norm_vec_kernel<T, 8><<<grid, threads, 0, st>>>(GN_ARGS)));
+#undef GN_ARGS
+    return jl_check_launch("gated_norm_kernel");
 }

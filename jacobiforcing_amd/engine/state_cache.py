@@ -16,7 +16,7 @@ import torch
 class RunSpec:
     """Memory one layer run needs.  kind "kv": ``k_width`` / ``v_width`` elements per cached token (all key/value heads side by
     side; ``v_width`` 0: the values are read out of the key rows, there is no second pool).  kind "state": a float tensor of
-    ``state_shape`` per slot.  kind None: nothing.  Beside either, ``tail_shape`` (when not empty) is a small float tensor per slot
+    ``state_shape`` per slot.  kind "kv+state": both (a layer whose mixer pairs attention with a recurrence).  kind None: nothing.  Beside either, ``tail_shape`` (when not empty) is a small float tensor per slot
     for what a layer carries from step to step whatever its mixer is (the last inputs of a short convolution); a layer that carries
     several such things of different shapes names them in ``tails`` (name -> shape per slot)."""
     kind: Optional[str]
@@ -38,12 +38,14 @@ class PagedStateCache:
         self.tail: List[Optional[torch.Tensor]] = []
         self.tails: List[Dict[str, torch.Tensor]] = []
         for s in specs:
-            kv = s.kind == "kv"
+            if s.kind not in (None, "kv", "state", "kv+state"):
+                raise ValueError(f"a layer run of kind {s.kind!r}")
+            kv, state = s.kind in ("kv", "kv+state"), s.kind in ("state", "kv+state")
             self.k.append(torch.zeros((tokens, s.k_width), dtype=dtype, device=device) if kv else None)
             self.v.append(torch.zeros((tokens, s.v_width), dtype=dtype, device=device) if kv and s.v_width else None)
             self.tail.append(torch.zeros((self.num_slots, *s.tail_shape), dtype=torch.float32, device=device)
                              if s.tail_shape and all(int(d) > 0 for d in s.tail_shape) else None)
-            self.state.append(torch.zeros((self.num_slots, *s.state_shape), dtype=torch.float32, device=device) if s.kind == "state" else None)
+            self.state.append(torch.zeros((self.num_slots, *s.state_shape), dtype=torch.float32, device=device) if state else None)
             self.tails.append({k: torch.zeros((self.num_slots, *shape), dtype=torch.float32, device=device)
                                for k, shape in s.tails.items() if shape and all(int(d) > 0 for d in shape)})
 

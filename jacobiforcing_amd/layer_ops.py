@@ -169,7 +169,10 @@ def add_rmsnorm(x: torch.Tensor, y: Optional[torch.Tensor], x0: Optional[torch.T
 
 
 def qk_norm_append(proj: torch.Tensor, cols: Tuple[int, int, int], H: int, G: int, D: int, Dv: int, wq: torch.Tensor, wk: torch.Tensor,
-                   eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor, kv_slot: torch.Tensor) -> torch.Tensor:
+                   eps: float, k_cache: torch.Tensor, v_cache: torch.Tensor, kv_slot: torch.Tensor, rot_dims: int = 0, pairing: int = N.JL_ROT_HALVES,
+                   batch: Optional["RaggedBatch"] = None, cos: Optional[torch.Tensor] = None, sin: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """RMS norm of q over all its heads together (and of k over its), with ``rot_dims`` the rotation of both by position behind it (needs
+    ``batch`` and its angle tables), keys / values appended to the pools.  Returns q [N, H*D]."""
     _dev(proj)
     n, ld = proj.shape
     dt = proj.dtype
@@ -177,9 +180,13 @@ def qk_norm_append(proj: torch.Tensor, cols: Tuple[int, int, int], H: int, G: in
     _need(wq.numel() == H * D and wk.numel() == G * D and wq.dtype == dt and wk.dtype == dt, "qk_norm_append: norm weights over the whole projections")
     _need(k_cache.dtype == dt and v_cache.dtype == dt and k_cache.is_contiguous() and v_cache.is_contiguous() and
           k_cache.shape[-1] == G * D and v_cache.shape[-1] == G * Dv and k_cache.shape[0] == v_cache.shape[0], "qk_norm_append: pools [tokens, G*D] / [tokens, G*Dv]")
+    if rot_dims:
+        _need(batch is not None and n == batch.N and rot_dims % 2 == 0 and 0 <= rot_dims <= D, "qk_norm_append: the rotation needs the batch and an even number of dimensions up to D")
+        _angle_tables(rot_dims, cos, sin, batch, "qk_norm_append")
     q = torch.empty((n, H * D), dtype=dt, device=proj.device)
     N.check_layers(N.layers().jl_qk_norm_append(_ptr(proj), _code(dt), n, ld, cols[0], cols[1], cols[2], H, G, D, Dv, _ptr(wq), _ptr(wk), float(eps),
-                                               _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(kv_slot), _stream(proj.device)), "jl_qk_norm_append")
+                                               _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(kv_slot), int(rot_dims), int(pairing), _ptr(batch.pos) if rot_dims else None,
+                                               _ptr(cos) if rot_dims else None, _ptr(sin) if rot_dims else None, _stream(proj.device)), "jl_qk_norm_append")
     return q
 
 
@@ -189,6 +196,14 @@ def _check_gate_sink(gate, sink, gate_per_head: bool, n: int, H: int, Dv: int, d
               f"{what}: gate [N, H*Dv], or [N, H] with one gate per head")
     if sink is not None:
         _need(sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == H, f"{what}: sink float [H]")
+
+
+def _attn_out(out: Optional[torch.Tensor], n: int, width: int, dtype: torch.dtype, device, what: str) -> torch.Tensor:
+    """The output matrix [n, width]: a new one, or the caller's column range of wider rows."""
+    if out is None:
+        return torch.empty((n, width), dtype=dtype, device=device)
+    _need(tuple(out.shape) == (n, width) and out.dtype == dtype and out.stride(1) == 1, f"{what}: out [N, H*Dv] of the output's dtype, contiguous along a row")
+    return out
 
 
 def attn_tile_rows(dtype: torch.dtype, H: int, G: int, D: int, Dv: int, k_ld: int = 0, v_ld: int = 0) -> int:
@@ -201,12 +216,15 @@ def attn_tile_rows(dtype: torch.dtype, H: int, G: int, D: int, Dv: int, k_ld: in
 def attn_window(q: torch.Tensor, gate: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor, batch: RaggedBatch,
                 H: int, G: int, D: int, Dv: int, scale: float, window: int, keep_first: int, rel: Optional[torch.Tensor],
                 lut: Optional[torch.Tensor], talk: Optional[torch.Tensor], value_heads: int = 0, float_out: bool = False,
-                sink: Optional[torch.Tensor] = None, gate_per_head: bool = False) -> torch.Tensor:
+                sink: Optional[torch.Tensor] = None, gate_per_head: bool = False, chunk: int = 0, softcap: float = 0.0, out_scale: float = 1.0,
+                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [N, H*D]; gate a [N, H*Dv] view (column range of the projection output, row stride free; [N, H] with ``gate_per_head``) or
     None.  ``sink`` float [H]: one more term exp(sink_h) in every softmax denominator of head h.  Returns [N, H*Dv].
     The pools may be column ranges of wider rows (``v_cache`` may be a view into ``k_cache``).  ``value_heads`` (0: G) < G: key head
     c reads value head c % value_heads — several score maps over the same values.  ``float_out``: float outputs from bfloat16
-    inputs (for what is subtracted or normalised next)."""
+    inputs (for what is subtracted or normalised next).  ``chunk`` > 0: a query sees the keys of its own run of ``chunk`` positions only (no
+    window beside it).  ``softcap`` > 0: scores pass softcap * tanh(s / softcap).  ``out_scale`` multiplies the outputs, which go to ``out``
+    (a column range of wider rows) when given."""
     _dev(q)
     dt = q.dtype
     n = q.shape[0]
@@ -224,13 +242,14 @@ def attn_window(q: torch.Tensor, gate: Optional[torch.Tensor], k_cache: torch.Te
             _need(t.dtype == torch.float32 and t.is_contiguous() and (shape is None or tuple(t.shape) == shape), "attn_window: float tables")
     if rel is not None:                                  # rel [rows, H] with lut [positions] -> row, or rel [positions, H] by distance itself
         _need(rel.shape[1] == H and (lut is None or lut.dtype == torch.int32), "attn_window: rel [rows, H] (+ int32 lut)")
+    _need(chunk <= 0 or (window <= 0 and keep_first <= 0), "attn_window: chunks exclude a window and kept first tokens")
     tq = attn_tile_rows(dt, H, G, D, Dv, k_ld, v_ld)
     tiles = batch.tiles(tq)
-    out = torch.empty((n, H * Dv), dtype=torch.float32 if float_out else dt, device=q.device)
+    out = _attn_out(out, n, H * Dv, torch.float32 if float_out else dt, q.device, "attn_window")
     # few tiles with many keys (decoding): share each tile's keys out over workgroups until the chip is full
     splits, scratch = 1, None
     if tq == 32 and tiles.shape[0] < ATTN_SPLIT_BELOW_TILES:
-        reach = batch.max_pos if window <= 0 else min(batch.max_pos, int(window) + int(keep_first) + tq)
+        reach = min(batch.max_pos, chunk + tq) if chunk > 0 else batch.max_pos if window <= 0 else min(batch.max_pos, int(window) + int(keep_first) + tq)
         splits = max(1, min(-(-reach // 64), ATTN_SPLIT_WORKGROUPS // tiles.shape[0], 64))
         if splits > 1:
             scratch = torch.empty((int(N.layers().jl_attn_scratch_floats(tiles.shape[0], n, H, Dv, splits)),), dtype=torch.float32, device=q.device)
@@ -244,7 +263,8 @@ def attn_window(q: torch.Tensor, gate: Optional[torch.Tensor], k_cache: torch.Te
                    scratch=scratch.data_ptr() if scratch is not None else None,
                    q_pack=q_pack.data_ptr() if q_pack is not None else None, k_ld=k_ld, v_ld=v_ld, Gv=Gv,
                    out_dtype=N.JL_OUT_F32 if float_out and dt != torch.float32 else N.JL_OUT_SAME,
-                   sink=sink.data_ptr() if sink is not None else None, gate_heads=int(gate_per_head))
+                   sink=sink.data_ptr() if sink is not None else None, gate_heads=int(gate_per_head), chunk=int(chunk), softcap=float(softcap),
+                   out_scale=float(out_scale), out_ld=out.stride(0))
     N.check_layers(N.layers().jl_attn_window(C.byref(a), _stream(q.device)), "jl_attn_window")
     return out
 
@@ -260,8 +280,9 @@ def attn_sweep_tile_rows(dtype: torch.dtype, H: int, G: int, D: int, Dv: int, k_
 
 def attn_sweep(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, batch: RaggedBatch, H: int, G: int, D: int, Dv: int, scale: float,
                window: int, value_heads: int = 0, float_out: bool = False, sink: Optional[torch.Tensor] = None,
-               gate: Optional[torch.Tensor] = None, gate_per_head: bool = False) -> torch.Tensor:
-    """Attention without bias or head mixing (``sink`` / ``gate`` as for ``attn_window``) in one sweep on the matrix cores: q [N, H*D] bfloat16, pools as for
+               gate: Optional[torch.Tensor] = None, gate_per_head: bool = False, chunk: int = 0, softcap: float = 0.0, out_scale: float = 1.0,
+               out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Attention without bias or head mixing (``sink`` / ``gate`` / ``chunk`` / ``softcap`` / ``out_scale`` / ``out`` as for ``attn_window``) in one sweep on the matrix cores: q [N, H*D] bfloat16, pools as for
     ``attn_window`` (column ranges of wider rows allowed); ``v_cache`` may be the first Dv columns of ``k_cache`` itself (one key
     head whose rows hold the values: the latent pool).  Returns [N, H*Dv].  Sizes as ``attn_sweep_tile_rows`` accepts them."""
     _dev(q)
@@ -275,8 +296,9 @@ def attn_sweep(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ba
     _check_gate_sink(gate, sink, gate_per_head, n, H, Dv, q.dtype, "attn_sweep")
     tq = attn_sweep_tile_rows(q.dtype, H, G, D, Dv, k_cache, v_cache, Gv)
     _need(tq > 0, f"attn_sweep: heads={H} kv_heads={G} dim={D} vdim={Dv} are not sizes of this kernel")
+    _need(chunk <= 0 or window <= 0, "attn_sweep: chunks exclude a window")
     tiles = batch.tiles(tq)
-    out = torch.empty((n, H * Dv), dtype=torch.float32 if float_out else q.dtype, device=q.device)
+    out = _attn_out(out, n, H * Dv, torch.float32 if float_out else q.dtype, q.device, "attn_sweep")
     # few tiles with many keys (decoding): share each tile's keys out over workgroups until the chip is full
     groups = tiles.shape[0] * G * -(-(H // G) // 32)
     splits, scratch = 1, None
@@ -287,7 +309,7 @@ def attn_sweep(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ba
         if wide > 0:
             tq, tiles = wide, batch.tiles(wide)
     elif groups < SWEEP_SPLIT_BELOW_GROUPS:
-        reach = batch.max_pos if window <= 0 else min(batch.max_pos, int(window) + tq)
+        reach = min(batch.max_pos, chunk + tq) if chunk > 0 else batch.max_pos if window <= 0 else min(batch.max_pos, int(window) + tq)
         splits = max(1, min(-(-reach // 128), SWEEP_SPLIT_WORKGROUPS // groups, 64))
         if splits > 1:
             scratch = torch.empty((int(N.layers().jl_attn_sweep_scratch_floats(tiles.shape[0], H, G, Dv, splits)),), dtype=torch.float32, device=q.device)
@@ -296,7 +318,8 @@ def attn_sweep(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ba
                    window=int(window), TQ=tq, dtype=_code(q.dtype), scale=float(scale), n_rows=n, k_ld=k_cache.stride(0), v_ld=v_cache.stride(0), Gv=Gv,
                    splits=splits, scratch=scratch.data_ptr() if scratch is not None else None,
                    out_dtype=N.JL_OUT_F32 if float_out else N.JL_OUT_SAME, sink=sink.data_ptr() if sink is not None else None,
-                   gate=gate.data_ptr() if gate is not None else None, gate_ld=gate.stride(0) if gate is not None else 0, gate_heads=int(gate_per_head))
+                   gate=gate.data_ptr() if gate is not None else None, gate_ld=gate.stride(0) if gate is not None else 0, gate_heads=int(gate_per_head),
+                   chunk=int(chunk), softcap=float(softcap), out_scale=float(out_scale), out_ld=out.stride(0))
     N.check_layers(N.layers().jl_attn_sweep(C.byref(a), _stream(q.device)), "jl_attn_sweep")
     return out
 
@@ -391,7 +414,8 @@ def moe_experts(h: torch.Tensor, router_logits: torch.Tensor, correction: Option
     return y
 
 
-ACT_GELU_TANH, ACT_CLAMPED_SWISH, ACT_SILU, ACT_GELU_ERF, ACT_NONE = N.JL_ACT_GELU_TANH, N.JL_ACT_CLAMPED_SWISH, N.JL_ACT_SILU, N.JL_ACT_GELU_ERF, N.JL_ACT_NONE
+ACT_GELU_TANH, ACT_CLAMPED_SWISH, ACT_SILU, ACT_GELU_ERF = N.JL_ACT_GELU_TANH, N.JL_ACT_CLAMPED_SWISH, N.JL_ACT_SILU, N.JL_ACT_GELU_ERF
+ACT_SIGMOID, ACT_NONE = N.JL_ACT_SIGMOID, N.JL_ACT_NONE
 
 
 def gated_act(z: torch.Tensor, g_col: int, u_col: int, F_: int, kind: int, limit: float = 0.0, alpha: float = 1.0, shift: float = 0.0,
@@ -454,6 +478,50 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, out_
     out = torch.empty((n, W), dtype=out_dtype, device=x.device) if out_dtype is not None else None
     N.check_layers(N.layers().jl_norm_add(_ptr(x), _ptr(y), _code(y.dtype), _ptr(g), float(eps), _ptr(out), _code(out_dtype or torch.float32), n, W,
                                          _stream(x.device)), "jl_norm_add")
+    return out
+
+
+def product_f32(a: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    """a [N, K] . w [M, K]^T with a float result [N, M] (not rounded to the operands' dtype): a product that becomes the residual stream."""
+    _dev(a)
+    return torch.mm(a, w.t()) if a.dtype == torch.float32 else torch.mm(a, w.t(), out_dtype=torch.float32)
+
+
+def sandwich_norm(x_in: torch.Tensor, y: Optional[torch.Tensor], w_post: Optional[torch.Tensor], eps: float, w_next: Optional[torch.Tensor] = None,
+                  out_dtype: Optional[torch.dtype] = None, add_row: Optional[torch.Tensor] = None, out: Optional[torch.Tensor] = None,
+                  plain: bool = False) -> Optional[torch.Tensor]:
+    """x_in (float [N, W], in place) += rms_norm(y) * w_post + add_row (each part optional: y [N, W] with its norm weight, add_row float [W]);
+    returns rms_norm(x_in) * w_next — or x_in itself with ``plain`` — in ``out_dtype`` or in ``out`` (a column range of wider rows); None with
+    neither."""
+    _dev(x_in)
+    n, W = x_in.shape
+    _need(x_in.dtype == torch.float32 and x_in.is_contiguous(), "sandwich_norm: x contiguous float32 [N, W]")
+    _need(y is None or (tuple(y.shape) == (n, W) and y.is_contiguous() and w_post is not None), "sandwich_norm: y [N, W] with its norm weight")
+    for w in (w_post, add_row, w_next):
+        _need(w is None or (w.dtype == torch.float32 and w.numel() == W and w.is_contiguous()), "sandwich_norm: weights and the added row are float [W]")
+    if out is not None:
+        _need(tuple(out.shape) == (n, W) and out.stride(1) == 1, "sandwich_norm: out [N, W], contiguous along a row")
+    elif out_dtype is not None:
+        out = torch.empty((n, W), dtype=out_dtype, device=x_in.device)
+    _need(out is None or plain or w_next is not None, "sandwich_norm: the second norm needs its weight")
+    N.check_layers(N.layers().jl_sandwich_norm(_ptr(x_in), _ptr(x_in), _ptr(y), _code(y.dtype) if y is not None else 0, _ptr(w_post), _ptr(add_row), float(eps),
+                                              _ptr(w_next), _ptr(out), _code(out.dtype) if out is not None else 0, out.stride(0) if out is not None else 0,
+                                              int(plain), n, W, _stream(x_in.device)), "jl_sandwich_norm")
+    return out
+
+
+def gated_norm(raw: torch.Tensor, gate: torch.Tensor, w: torch.Tensor, eps: float, act: int, gate_first: bool, parts: int = 1, scale: float = 1.0,
+               out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """raw float [N, C] and its gate [N, C] (a column range of a product, row stride free): rms_norm over ``parts`` equal parts of the row of
+    raw * act(gate) (``gate_first``), or of raw with act(gate) on the result; times w (float [C]) and ``scale``.  [N, C] of gate's dtype, in
+    ``out`` (a column range of wider rows) when given."""
+    _dev(raw)
+    n, C_ = raw.shape
+    _need(raw.dtype == torch.float32 and raw.is_contiguous() and tuple(gate.shape) == (n, C_) and gate.stride(1) == 1, "gated_norm: raw float [N, C], gate [N, C]")
+    _need(w.dtype == torch.float32 and w.numel() == C_ and w.is_contiguous() and parts >= 1 and C_ % parts == 0, "gated_norm: w float [C], parts that divide C")
+    out = _attn_out(out, n, C_, gate.dtype, raw.device, "gated_norm")
+    N.check_layers(N.layers().jl_gated_norm(_ptr(raw), _ptr(gate), _code(gate.dtype), gate.stride(0), _ptr(w), float(eps), int(act), int(gate_first), float(scale),
+                                           _ptr(out), out.stride(0), n, C_, int(parts), _stream(raw.device)), "jl_gated_norm")
     return out
 
 
@@ -662,9 +730,10 @@ def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
     return z
 
 
-def short_conv(x: torch.Tensor, col: int, C_: int, w: torch.Tensor, batch: RaggedBatch, tail: Optional[torch.Tensor], act: int = N.JL_ACT_SILU) -> torch.Tensor:
-    """act(causal depthwise convolution over time, per request) of the columns col .. col + C_ of x [N, ld], with w [C_, taps]; float
-    [N, C_].  ``tail`` float [slots, taps - 1, C_] carries every request's last inputs from step to step (updated here)."""
+def short_conv(x: torch.Tensor, col: int, C_: int, w: torch.Tensor, batch: RaggedBatch, tail: Optional[torch.Tensor], act: int = N.JL_ACT_SILU,
+               bias: Optional[torch.Tensor] = None, out_dtype: torch.dtype = torch.float32) -> torch.Tensor:
+    """act(bias + causal depthwise convolution over time, per request) of the columns col .. col + C_ of x [N, ld], with w [C_, taps]; [N, C_]
+    of ``out_dtype`` (float, or x's).  ``tail`` float [slots, taps - 1, C_] carries every request's last inputs from step to step (updated here)."""
     _dev(x)
     n, ld = x.shape
     taps = w.shape[1]
@@ -673,9 +742,11 @@ def short_conv(x: torch.Tensor, col: int, C_: int, w: torch.Tensor, batch: Ragge
     if taps > 1:
         _need(tail is not None and tail.dtype == torch.float32 and tail.is_contiguous() and tuple(tail.shape[1:]) == (taps - 1, C_) and
               batch.max_slot < tail.shape[0], "short_conv: tail float [slots, taps - 1, C] with the batch's slots")
-    out = torch.empty((n, C_), dtype=torch.float32, device=x.device)
-    N.check_layers(N.layers().jl_short_conv(_ptr(x), _code(x.dtype), ld, col, _ptr(w), _ptr(batch.row_req), _ptr(batch.seq), batch.B, max(batch.counts),
-                                           _ptr(tail), n, C_, taps, int(act), _ptr(out), _stream(x.device)), "jl_short_conv")
+    _need(bias is None or (bias.dtype == x.dtype and bias.numel() == C_ and bias.is_contiguous()), "short_conv: bias [C] of x's dtype")
+    _need(out_dtype in (torch.float32, x.dtype), "short_conv: the output is float or of x's dtype")
+    out = torch.empty((n, C_), dtype=out_dtype, device=x.device)
+    N.check_layers(N.layers().jl_short_conv(_ptr(x), _code(x.dtype), ld, col, _ptr(w), _ptr(bias), _ptr(batch.row_req), _ptr(batch.seq), batch.B, max(batch.counts),
+                                           _ptr(tail), n, C_, taps, int(act), _ptr(out), _code(out_dtype), _stream(x.device)), "jl_short_conv")
     return out
 
 
@@ -700,4 +771,30 @@ def delta_rule(qkv: torch.Tensor, cols: Tuple[int, int, int], proj: torch.Tensor
     N.check_layers(N.layers().jl_delta_rule(_ptr(qkv), N.JL_F32, qkv.shape[1], cols[0], cols[1], cols[2], _ptr(proj), _code(proj.dtype), ld, pcols[0], pcols[1],
                                            pcols[2], _ptr(a_log), _ptr(dt_bias), _ptr(norm_w), _ptr(batch.seq), batch.B, n, H, G, D, Dv, float(unit_eps),
                                            float(q_scale), float(eps), _ptr(state), _ptr(raw), _ptr(out), _stream(proj.device)), "jl_delta_rule")
+    return out
+
+
+def linear_scan(src: torch.Tensor, cols: Tuple[int, int, int], batch: RaggedBatch, H: int, G: int, D: int, Dv: int, state: torch.Tensor, act: int = N.JL_ACT_NONE,
+                decay: Optional[torch.Tensor] = None, dt: Optional[torch.Tensor] = None, a_log: Optional[torch.Tensor] = None,
+                dt_bias: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Linear recurrence S <- a S + k (u v)^T, o = S^T q + skip v per head.  src [N, ld] holds q, k (G*D each) and v (H*Dv) at ``cols``, which pass
+    ``act`` on the way in.  ``decay`` float [H]: a = decay, u = 1; else u = softplus(dt + dt_bias), a = exp(-exp(a_log) u) with dt [N, H] (row
+    stride free, src's dtype), a_log / dt_bias float [H].  skip float [H] or None.  state [slots, H, D, Dv] float, updated in place.  Returns
+    float [N, H*Dv]."""
+    _dev(src)
+    n, ld = src.shape
+    _need(src.stride(1) == 1 and n == batch.N and H % G == 0 and max(cols[0], cols[1]) + G * D <= ld and cols[2] + H * Dv <= ld, "linear_scan: columns of the batch's rows")
+    _need(state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (H, D, Dv) and batch.max_slot < state.shape[0],
+          "linear_scan: state float [slots, H, D, Dv] with the batch's slots")
+    _need(decay is not None or (dt is not None and a_log is not None and dt_bias is not None), "linear_scan: fixed decays, or dt with a_log and dt_bias")
+    for t in (decay, a_log, dt_bias, skip):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == H), "linear_scan: per-head constants are float [H]")
+    if decay is None:
+        _need(tuple(dt.shape) == (n, H) and dt.stride(1) == 1 and dt.dtype == src.dtype, "linear_scan: dt [N, H] of src's dtype")
+    out = torch.empty((n, H * Dv), dtype=torch.float32, device=src.device)
+    p = lambda t: t.data_ptr() if t is not None else None
+    a = N.ScanArgs(src=p(src), dt=p(dt) if decay is None else None, decay=p(decay), A_log=p(a_log), dt_bias=p(dt_bias), skip=p(skip), seq=p(batch.seq), state=p(state), out=p(out),
+                   ld=src.stride(0), dt_ld=dt.stride(0) if decay is None else 0, N=n, q_col=cols[0], k_col=cols[1], v_col=cols[2], dt_col=0, dtype=_code(src.dtype),
+                   act=int(act), B=batch.B, H=H, G=G, D=D, Dv=Dv)
+    N.check_layers(N.layers().jl_linear_scan(C.byref(a), _stream(src.device)), "jl_linear_scan")
     return out

@@ -16,6 +16,7 @@ MODEL_REGISTRY = {
     "Vumalix": ("jacobiforcing_amd.modeling.vumalix", "VumalixConfig", "ragged"),
     "Bamanex": ("jacobiforcing_amd.modeling.bamanex", "BamanexConfig", "ragged"),
     "Mikipel": ("jacobiforcing_amd.modeling.mikipel", "MikipelConfig", "ragged"),
+    "Safisun": ("jacobiforcing_amd.modeling.safisun", "SafisunConfig", "ragged"),
 }
 
 
