@@ -284,8 +284,9 @@ JL_API int jl_delta_rule(const void *qkv, int qkv_dtype, int64_t qkv_ld, int32_t
  * in dt [N, dt_ld] of `dtype`; skip float [H] or null.  state [slots, H, D, Dv] float: a request with pos0 == 0 starts from zero (its
  * slot's old content is ignored); the final state is written back.  out float [N, H*Dv].  D <= 256.
  * `chunks` 0: every request's rows in one scan.  `chunks` > 0 (bfloat16, long portions): the portions are cut into `chunks` pieces that
- * run side by side on the matrix cores — chunk_rec [chunks, 4] int32 {row0, count, pos0, piece}, req [B, 4] int32 {first piece, pieces,
- * pos0, slot}, scratch of chunks * H * (D * Dv + 1) floats; sizes as jl_linear_scan_chunked_ok accepts them. */
+ * run side by side on the matrix cores — chunk_rec [chunks, 4] int32 {row0, count, slot, 1 for a request's last piece}, every piece but the
+ * last a multiple of 64 rows, a request's pieces consecutive; req [B, 4] int32 {first piece, pieces, pos0, slot}; scratch of
+ * chunks * H * (D * Dv + 1) floats; sizes as jl_linear_scan_chunked_ok accepts them, rows and columns in multiples of four elements. */
 typedef struct {
     const void *src; const void *dt; const float *decay; const float *A_log; const float *dt_bias; const float *skip;
     const int32_t *seq; float *state; float *out; const int32_t *chunk_rec; const int32_t *req; float *scratch;

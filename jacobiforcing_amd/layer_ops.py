@@ -21,6 +21,7 @@ ATTN_MAX_HEADS_ONE_LAUNCH, ATTN_MAX_VALUE_WIDTH = 16, 128   # what the matrix-co
 SWEEP_SPLIT_BELOW_GROUPS, SWEEP_SPLIT_WORKGROUPS = 512, 2048   # one-sweep attention: its workgroups are small (4 wavefronts, <= 32 rows)
 SWEEP_WIDE_ROWS_PER_REQUEST = 16   # one-sweep attention: from this many tokens per request on average a step takes the 128-row tiles
 RETENTION_CHUNK = 64          # tokens per chunk when a long portion's recurrence is cut into chunks that run side by side
+SCAN_PIECES_FROM, SCAN_WORKGROUPS = 32, 512     # linear recurrence: portions from this many tokens on run in pieces on the matrix cores; workgroups to aim at
 DELTA_COLUMNS_FROM = 32       # delta rule: from this many tokens in a request's portion on, the state's columns are shared out over wavefronts
 
 
@@ -68,6 +69,7 @@ class RaggedBatch:
     max_pos: int
     max_page: int
     max_slot: int
+    slots: List[int]
     _tiles: dict
 
     @classmethod
@@ -94,7 +96,7 @@ class RaggedBatch:
                    row_req=torch.from_numpy(np.repeat(np.arange(B, dtype=np.int32), np.asarray(counts, dtype=np.int64))).to(dev),
                    pos=torch.from_numpy(row_pos).to(dev),
                    page_size=int(page_size), max_pos=max(int(s) + int(c) for s, c in zip(starts, counts)), max_page=int(bt.max()),
-                   max_slot=int(max(slots)), _tiles={})
+                   max_slot=int(max(slots)), slots=list(map(int, slots)), _tiles={})
 
     def chunks(self, size: int):
         """A portion of at least two chunks is cut into chunks of ``size`` tokens that the recurrent layers run side by side.
@@ -115,6 +117,20 @@ class RaggedBatch:
                 plan = (torch.from_numpy(rec).to(dev), torch.from_numpy(np.ascontiguousarray(rec[:, 1])).to(dev),
                         torch.from_numpy(np.asarray(req, dtype=np.int32).reshape(-1, 4)).to(dev))
             self._tiles[key] = plan
+        return self._tiles[key]
+
+    def pieces(self, size: int):
+        """Every request's portion cut into pieces of ``size`` tokens: (piece records [pieces, 4] int32 {row0, count, slot, 1 for a request's
+        last piece}, request records [B, 4] int32 {first piece, pieces, pos0, slot}), on the device."""
+        key = ("pieces", size)
+        if key not in self._tiles:
+            rec, req, r0 = [], [], 0
+            for c, s, sl in zip(self.counts, self.starts, self.slots):
+                req.append((len(rec), -(-c // size), s, sl))
+                rec += [(r0 + o, min(size, c - o), sl, int(o + size >= c)) for o in range(0, c, size)]
+                r0 += c
+            both = torch.tensor(rec + req, dtype=torch.int32, device=self.seq.device).reshape(-1, 4)
+            self._tiles[key] = (both[:len(rec)], both[len(rec):])
         return self._tiles[key]
 
     def tiles(self, tq: int) -> torch.Tensor:
@@ -796,5 +812,12 @@ def linear_scan(src: torch.Tensor, cols: Tuple[int, int, int], batch: RaggedBatc
     a = N.ScanArgs(src=p(src), dt=p(dt) if decay is None else None, decay=p(decay), A_log=p(a_log), dt_bias=p(dt_bias), skip=p(skip), seq=p(batch.seq), state=p(state), out=p(out),
                    ld=src.stride(0), dt_ld=dt.stride(0) if decay is None else 0, N=n, q_col=cols[0], k_col=cols[1], v_col=cols[2], dt_col=0, dtype=_code(src.dtype),
                    act=int(act), B=batch.B, H=H, G=G, D=D, Dv=Dv)
+    if (max(batch.counts) >= SCAN_PIECES_FROM and not os.environ.get("JL_SCAN_NO_PIECES") and a.ld % 4 == 0 and all(c % 4 == 0 for c in cols) and    # A/B switch for measurements
+            N.layers().jl_linear_scan_chunked_ok(a.dtype, D, Dv)):
+        # long portions: pieces side by side on the matrix cores, as many as fill the chip, each at least one group of 64 tokens
+        size = 64 * max(1, min(8, n * H * -(-Dv // 64) // (SCAN_WORKGROUPS * 64)))
+        rec, req = batch.pieces(size)
+        scratch = torch.empty((rec.shape[0] * H * (D * Dv + 1),), dtype=torch.float32, device=src.device)
+        a.chunk_rec, a.req, a.scratch, a.chunks = p(rec), p(req), p(scratch), rec.shape[0]
     N.check_layers(N.layers().jl_linear_scan(C.byref(a), _stream(src.device)), "jl_linear_scan")
     return out
