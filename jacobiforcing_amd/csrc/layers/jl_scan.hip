@@ -8,6 +8,12 @@
 // columns): two adjacent lanes per column, each with DMAX / 2 consecutive rows in registers.  Rows of S are read and written as 128
 // consecutive bytes.  Eight tokens at a time go through LDS; the next group's inputs travel while the current one is worked on.
 constexpr int SC_TT = 8, SC_COLS = 32;
+// silu in the activations' dtype: both forms of the recurrence see the same q, k and v, however a prompt is cut
+template <typename T> __device__ __forceinline__ float silu_as(float z) {
+    T t;
+    st_f(&t, silu_f(z));
+    return ld_f(&t);
+}
 
 template <typename T, int DMAX>
 __global__ __launch_bounds__(64) void scan_kernel(jl_scan_args a) {
@@ -54,8 +60,8 @@ __global__ __launch_bounds__(64) void scan_kernel(jl_scan_args a) {
         for (int i = 0; i < PRE; ++i) {
             const int e = i * 64 + lane, tt = e / DMAX, d = e - tt * DMAX;
             if (tt < nt) {
-                qs[at(tt, d)] = act ? silu_f(pq[i]) : pq[i];
-                ks[at(tt, d)] = act ? silu_f(pk[i]) : pk[i];
+                qs[at(tt, d)] = act ? silu_as<T>(pq[i]) : pq[i];
+                ks[at(tt, d)] = act ? silu_as<T>(pk[i]) : pk[i];
             }
         }
         if (lane < nt) {
@@ -65,7 +71,7 @@ __global__ __launch_bounds__(64) void scan_kernel(jl_scan_args a) {
         }
         float v[SC_TT];
 #pragma unroll
-        for (int tt = 0; tt < SC_TT; ++tt) v[tt] = act ? silu_f(pv[tt]) : pv[tt];
+        for (int tt = 0; tt < SC_TT; ++tt) v[tt] = act ? silu_as<T>(pv[tt]) : pv[tt];
         __syncthreads();
         if (t0 + SC_TT < cnt) fetch(t0 + SC_TT);                // in flight while this group's steps run
 #pragma unroll
@@ -111,14 +117,15 @@ template <typename T> static int scan_launch(const jl_scan_args &a, hipStream_t 
 // from), outputs (CH_OUT; the last piece leaves the request's final state in its slot).  A workgroup of four wavefronts owns 64 columns of one
 // head's state and walks its piece's groups with the state in accumulators; the next group's rows travel while the current one is multiplied.
 // q, k and v enter the products as bfloat16 (what the projection, the convolution and their activation give); everything else stays float
-// and crosses the matrix cores as the sum of TWO bfloat16 numbers (16 bits of mantissa): the state, the decayed weights of a pair, the decayed
-// values.  Accumulator r of lane l of a 32 x 32 product is row 8 (r / 4) + 4 (l / 32) + r % 4, column l % 32; lane l supplies row (A) or column
+// and crosses the matrix cores as the sum of THREE bfloat16 numbers, which hold all 24 bits of it: the state, the decayed weights of a pair,
+// the decayed values.  Accumulator r of lane l of a 32 x 32 product is row 8 (r / 4) + 4 (l / 32) + r % 4, column l % 32; lane l supplies row (A) or column
 // (B) l % 32 with depths 8 (l / 32) .. + 7 of a 16-deep step.
 typedef __bf16 ch_bf16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 ch_bf16x4 __attribute__((ext_vector_type(4)));
 typedef float ch_f32x4 __attribute__((ext_vector_type(4)));
 typedef float ch_f32x16 __attribute__((ext_vector_type(16)));
 constexpr int CH_T = 64, CH_C = 64, CH_THREADS = 256, CH_TROW = CH_T, CH_PROW = CH_T + 8;
+constexpr int CH_TERMS = 3;
 constexpr int CH_OUT = 0, CH_LOCAL = 1;
 
 __device__ __forceinline__ ch_f32x16 ch_mfma(const bf16_t *a, const bf16_t *b, ch_f32x16 c) {
@@ -128,10 +135,14 @@ __device__ __forceinline__ uint2 ch_round4(const float (&v)[4]) {
     const ch_f32x4 f = {v[0], v[1], v[2], v[3]};
     return __builtin_bit_cast(uint2, __builtin_convertvector(f, ch_bf16x4));
 }
-__device__ __forceinline__ void ch_split4(const float (&v)[4], uint2 &hi, uint2 &lo) {
-    hi = ch_round4(v);
-    const float r[4] = {v[0] - __uint_as_float(hi.x << 16), v[1] - __uint_as_float(hi.x & 0xffff0000u), v[2] - __uint_as_float(hi.y << 16), v[3] - __uint_as_float(hi.y & 0xffff0000u)};
-    lo = ch_round4(r);
+// four floats as the sum of CH_TERMS bfloat16 numbers each, term x of them at dst + x * stride
+__device__ __forceinline__ void ch_split4(float (&v)[4], bf16_t *dst, int stride) {
+#pragma unroll
+    for (int x = 0; x < CH_TERMS; ++x) {
+        const uint2 w = ch_round4(v);
+        *(uint2 *)(dst + x * stride) = w;
+        v[0] -= __uint_as_float(w.x << 16); v[1] -= __uint_as_float(w.x & 0xffff0000u); v[2] -= __uint_as_float(w.y << 16); v[3] -= __uint_as_float(w.y & 0xffff0000u);
+    }
 }
 __device__ __forceinline__ uint2 ch_silu4(uint2 w) {
     float v[4] = {__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16), __uint_as_float(w.y & 0xffff0000u)};
@@ -151,13 +162,13 @@ __device__ __forceinline__ void ch_turn(bf16_t *dst, int row, int t, uint2 a, ui
 }
 
 static constexpr size_t ch_lds_bytes(int DP, bool out) {
-    return 2 * ((size_t)DP * CH_TROW + CH_C * CH_TROW + 2 * CH_C * CH_PROW + (out ? 2 * CH_T * (DP + 8) + 2 * CH_C * (DP + 8) : 0)) + 3 * CH_T * 4;
+    return 2 * ((size_t)DP * CH_TROW + CH_C * CH_TROW + CH_TERMS * CH_T * CH_PROW + (out ? 2 * CH_T * (DP + 8) + CH_TERMS * CH_C * (DP + 8) : 0)) + 3 * CH_T * 4;
 }
 
 template <int DP, int MODE>
 __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
-    constexpr int QROW = DP + 8, UD = DP / 4, KIT = 32 * UD / CH_THREADS, VIT = 2, NS = DP >= 64 ? DP / 64 : 1;
+    constexpr int QROW = DP + 8, UD = DP / 4, KIT = 32 * UD / CH_THREADS, VIT = 2, NS = DP >= 64 ? DP / 64 : 1, PT = CH_T * CH_PROW, ST = CH_C * QROW;
     constexpr bool OUT = MODE == CH_OUT;
     const int H = a.H, D = a.D, Dv = a.Dv;
     const int piece = blockIdx.x, h = blockIdx.y, kh = h / (H / a.G), c_base = blockIdx.z * CH_C;
@@ -165,10 +176,10 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
     if (cnt <= 0 || (!OUT && last)) return;
     bf16_t *KT = (bf16_t *)smem;                                    // [DP][64] keys, turned
     bf16_t *VT = KT + DP * CH_TROW;                                 // [64][64] values, turned
-    bf16_t *Phi = VT + CH_C * CH_TROW, *Plo = Phi + CH_T * CH_PROW;    // [64][72] weights of the pairs; then the decayed values (turned)
-    bf16_t *Qs = Plo + CH_T * CH_PROW, *Ks = Qs + CH_T * QROW;      // [64][DP + 8]
-    bf16_t *Shi = Ks + CH_T * QROW, *Slo = Shi + CH_C * QROW;       // [64][DP + 8] the state, turned
-    float *Ls = (float *)(OUT ? Slo + CH_C * QROW : Qs);            // [64] running log decay
+    bf16_t *Ps = VT + CH_C * CH_TROW;                               // terms x [64][72] weights of the pairs; then the decayed values (turned)
+    bf16_t *Qs = Ps + CH_TERMS * PT, *Ks = Qs + CH_T * QROW;        // [64][DP + 8]
+    bf16_t *Ss = Ks + CH_T * QROW;                                  // terms x [64][DP + 8] the state, turned
+    float *Ls = (float *)(OUT ? Ss + CH_TERMS * ST : Qs);           // [64] running log decay
     float *us = Ls + CH_T, *es = us + CH_T;                         // [64] u; [64] exp(L_end - L) u
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, l32 = lane & 31, hi = lane >> 5, w0 = wave & 1, w1 = wave >> 1;
     const bf16_t *src = (const bf16_t *)a.src, *dtp = (const bf16_t *)a.dt;
@@ -187,18 +198,14 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
             const int d = 32 * (w1 + 2 * x) + 8 * (r >> 2) + 4 * hi + (r & 3);
             S[x][r] = (OUT && d < D && sc < Dv) ? sp[(int64_t)d * Dv + sc] : 0.f;
         }
-    auto state_out = [&]() {                                        // the state in LDS, as two bfloat16 numbers each
+    auto state_out = [&]() {                                        // the state in LDS
 #pragma unroll
         for (int x = 0; x < NS; ++x) {
             if (32 * (w1 + 2 * x) >= DP) continue;
 #pragma unroll
             for (int g = 0; g < 4; ++g) {
-                const float v[4] = {S[x][4 * g], S[x][4 * g + 1], S[x][4 * g + 2], S[x][4 * g + 3]};
-                uint2 vh, vl;
-                ch_split4(v, vh, vl);
-                const int o = (32 * w0 + l32) * QROW + 32 * (w1 + 2 * x) + 8 * g + 4 * hi;
-                *(uint2 *)(Shi + o) = vh;
-                *(uint2 *)(Slo + o) = vl;
+                float v[4] = {S[x][4 * g], S[x][4 * g + 1], S[x][4 * g + 2], S[x][4 * g + 3]};
+                ch_split4(v, Ss + (32 * w0 + l32) * QROW + 32 * (w1 + 2 * x) + 8 * g + 4 * hi, ST);
             }
         }
     };
@@ -300,10 +307,7 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
                     float v[4];
 #pragma unroll
                     for (int x = 0; x < 4; ++x) v[x] = j0 + x <= i ? s[4 * g + x] * (__expf(li - Ls[j0 + x]) * us[j0 + x]) : 0.f;
-                    uint2 vh, vl;
-                    ch_split4(v, vh, vl);
-                    *(uint2 *)(Phi + i * CH_PROW + j0) = vh;
-                    *(uint2 *)(Plo + i * CH_PROW + j0) = vl;
+                    ch_split4(v, Ps + i * CH_PROW + j0, PT);
                 }
             }
             __syncthreads();
@@ -314,8 +318,8 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
                 const int ai = (32 * w1 + l32) * QROW + 8 * hi, bi = (32 * w0 + l32) * QROW + 8 * hi;
 #pragma unroll
                 for (int kk = 0; kk < DP; kk += 16) {
-                    o = ch_mfma(Qs + ai + kk, Shi + bi + kk, o);
-                    o = ch_mfma(Qs + ai + kk, Slo + bi + kk, o);
+#pragma unroll
+                    for (int x = 0; x < CH_TERMS; ++x) o = ch_mfma(Qs + ai + kk, Ss + x * ST + bi + kk, o);
                 }
 #pragma unroll
                 for (int r = 0; r < 16; ++r) o[r] *= __expf(Ls[32 * w1 + 8 * (r >> 2) + 4 * hi + (r & 3)]);
@@ -323,8 +327,8 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
                 for (int kk = 0; kk < CH_T; kk += 16) {
                     if (kk >= 32 && w1 == 0) continue;              // no key of the second half is visible to the first half's queries
                     const bf16_t *vp = VT + ch_tr(32 * w0 + l32, kk + 8 * hi);
-                    o = ch_mfma(Phi + (32 * w1 + l32) * CH_PROW + kk + 8 * hi, vp, o);
-                    o = ch_mfma(Plo + (32 * w1 + l32) * CH_PROW + kk + 8 * hi, vp, o);
+#pragma unroll
+                    for (int x = 0; x < CH_TERMS; ++x) o = ch_mfma(Ps + x * PT + (32 * w1 + l32) * CH_PROW + kk + 8 * hi, vp, o);
                 }
                 if (sc < Dv) {
 #pragma unroll
@@ -350,10 +354,7 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
                 ld4_f(VT + o, v);
 #pragma unroll
                 for (int y = 0; y < 4; ++y) v[y] *= es[t + y];
-                uint2 vh, vl;
-                ch_split4(v, vh, vl);
-                *(uint2 *)(Phi + o) = vh;
-                *(uint2 *)(Plo + o) = vl;
+                ch_split4(v, Ps + o, PT);
             }
         }
         __syncthreads();
@@ -368,8 +369,8 @@ __global__ __launch_bounds__(CH_THREADS) void scan_chunk_kernel(jl_scan_args a) 
                 for (int kk = 0; kk < CH_T; kk += 16) {
                     const bf16_t *kp = KT + ch_tr(32 * (w1 + 2 * x) + l32, kk + 8 * hi);
                     const int o = ch_tr(32 * w0 + l32, kk + 8 * hi);
-                    S[x] = ch_mfma(kp, Phi + o, S[x]);
-                    S[x] = ch_mfma(kp, Plo + o, S[x]);
+#pragma unroll
+                    for (int y = 0; y < CH_TERMS; ++y) S[x] = ch_mfma(kp, Ps + y * PT + o, S[x]);
                 }
             }
             if (OUT && t0 + CH_T < cnt) state_out();                // its readers of this group are two barriers behind

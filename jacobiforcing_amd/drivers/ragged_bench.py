@@ -1,9 +1,9 @@
 #!/usr/bin/env python3
-"""Prefill and decode throughput of a ragged model family (Lokizen, Vumalix, Bamanex, Mikipel) at sizes that resemble a real model's
+"""Prefill and decode throughput of a ragged model family (Lokizen, Vumalix, Bamanex, Mikipel, Safisun) at sizes that resemble a real model's
 layers, beside the package's closest existing model at equal width, depth, head sizes and active feed-forward width (Lokizen beside
-Qwen2; Vumalix, Bamanex and Mikipel beside Lokizen and Qwen2) — random weights, synthetic tokens.
+Qwen2; Vumalix, Bamanex, Mikipel and Safisun beside Lokizen and Qwen2) — random weights, synthetic tokens.
 
-    python -m jacobiforcing_amd.drivers.ragged_bench [--design lokizen|vumalix|bamanex|mikipel] [--sizes small,medium] [--kernels]
+    python -m jacobiforcing_amd.drivers.ragged_bench [--design lokizen|vumalix|bamanex|mikipel|safisun] [--sizes small,medium] [--kernels]
     python bench.py --design lokizen            (the same, as one JSON line)
 
 Per size: prefill = whole prompts in one step (tokens / s), decode = one token for each of ``--decode-batch`` requests at a
@@ -533,6 +533,140 @@ def kernel_table_mikipel(s, prompts, prompt_len, decode_batch, context, dtype=to
     return out
 
 
+# Safisun at Lokizen's widths, depths, head counts and head sizes: lightning, Mamba-2, parallel (attention beside lightning), Mamba-2 in turn, a dense
+# feed-forward of the experts' active width in every layer, one pass of the loop over the whole stack (its product in front, no extra depth);
+# Mamba-2 with heads of 64 over a state of 128, four taps, as many channels as the other mixers; chunks as long as Lokizen's window
+def safisun_config(s):
+    from ..modeling.safisun import SafisunConfig
+    H, G, D, W = s["heads"], s["kv"], s["dim"], s["width"]
+    light = {"heads": H, "dim": D, "vdim": D, "decay": [1 - 2.0 ** (-5 - 3 * h / H) for h in range(H)]}
+    lig = {"type": "lightning", "mixer": light}
+    mam = {"type": "mamba2", "mixer": {"heads": H * D // 64, "vdim": 64, "state": 128, "groups": 1, "norm_groups": 1, "conv": 4}}
+    par = {"type": "parallel", "mixer": {"left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "softcap": 50.0, "mask": {"size": s["window"]},
+                                                  "rot": {"dims": D // 2, "base": 1e6}}, "right": light, "left_scale": 0.6, "right_scale": 1.1}}
+    order = [lig, mam, par, mam]
+    return SafisunConfig.from_dict({"architecture": "Safisun", "vocab": s["vocab"], "width": W, "norm": {"eps": 1e-5}, "loop": {"start": 0, "stop": s["layers"], "times": 1},
+                                    "layers": [dict(order[i % 4], mlp={"kind": "dense", "ff": s["top"] * s["ff"]}) for i in range(s["layers"])]})
+
+
+def bench_safisun(s, prompts, prompt_len, decode_batch, context, dtype=torch.bfloat16):
+    from ..modeling.safisun import random_model
+    model = random_model(safisun_config(s), "cuda", dtype, max_positions=max(prompt_len, context) + 64)
+    # decode at a chunk's last position: the attention has its whole chunk to read (one position on it would see itself alone)
+    return bench_ragged(model, s["vocab"], prompts, prompt_len, decode_batch, context - 1)
+
+
+def kernel_table_safisun(s, prompts, prompt_len, decode_batch, context, dtype=torch.bfloat16):
+    """Safisun's layer kernels alone at the size's shapes, prefill and decode, each beside the like kernel of the closest model (Lokizen's
+    residual + norm launch, its retention, its whole-projection q/k norm, its windowed attention; Bamanex's attention with sink and gate;
+    Mikipel's delta rule; Vumalix's convolution; Qwen2's SwiGLU launch)."""
+    from .. import layer_ops as LO
+    from .. import ops
+    dev = "cuda"
+    H, G, D, W, top, ff, win = s["heads"], s["kv"], s["dim"], s["width"], s["top"], s["ff"], s["window"]
+    page, es = 64, 2
+    per = -(-(max(prompt_len, context) + 1) // page)
+    slots = max(prompts, decode_batch)
+    tables = [list(range(b * per, (b + 1) * per)) for b in range(slots)]
+    g = torch.Generator().manual_seed(0)
+    rnd = lambda *sh: torch.randn(*sh, generator=g).to(dev).to(dtype)
+    kc, vc = rnd(slots * per * page, G * D), rnd(slots * per * page, G * D)
+    a = torch.arange(max(prompt_len, context) + 8, dtype=torch.float32, device=dev).view(-1, 1) * torch.rand(D // 2, device=dev).view(1, -1)
+    cos, sin = a.cos().contiguous(), a.sin().contiguous()
+    hcos, hsin = cos[:, :D // 4].contiguous(), sin[:, :D // 4].contiguous()
+    state, decay = torch.zeros((slots, H, D, D), device=dev), torch.full((H,), 0.99, device=dev)
+    MH, MD, MN = H * D // 64, 64, 128
+    C_, taps = H * D + 2 * MN, 4
+    mstate, ctail, vtail = torch.zeros((slots, MH, MN, MD), device=dev), torch.zeros((slots, taps - 1, C_), device=dev), torch.zeros((slots, taps - 1, W), device=dev)
+    a_log, dt_bias, skip = torch.zeros(MH, device=dev), torch.zeros(MH, device=dev), torch.ones(MH, device=dev)
+    da_log, dnw = torch.zeros(H, device=dev), torch.ones(D, device=dev)
+    sink, ones = torch.zeros(H, device=dev), torch.ones(H * D, device=dev)
+    out = {}
+
+    def row(name, secs, nbytes, flops, peak):
+        bound = max(nbytes / HBM_BPS, flops / peak)
+        out[name] = {"us": round(1e6 * secs, 1), "MB": round(nbytes / 1e6, 2), "GFLOP": round(flops / 1e9, 2), "roofline_fraction": round(bound / secs, 4)}
+
+    for phase, B, T, start in (("prefill", prompts, prompt_len, 0), ("decode", decode_batch, 1, context - 1)):
+        n = B * T
+        batch = LO.RaggedBatch.build([T] * B, [start] * B, list(range(B)), tables[:B], page, dev)
+        chunked = B * sum((start + t) % win + 1 for t in range(T))                                 # visible (query, key) pairs per head
+        windowed = B * sum(min(start + t + 1, win) for t in range(T))
+        span_k, span_w = B * max((start + t) % win + 1 for t in range(T)) if T == 1 else B * T, B * min(start + T, win + T)      # pool rows a launch has to read once
+        x, y, wf, wn = torch.randn(n, W, device=dev), rnd(n, W), torch.randn(W, device=dev), rnd(W)
+        # output norm + residual update + next norm  |  Lokizen: update + one norm
+        row(f"{phase}.sandwich_norm", timed(lambda: LO.sandwich_norm(x, y, wf, 1e-5, wf, dtype)), n * W * (4 + 4 + es + es), 8.0 * n * W, VECTOR_FLOPS)
+        row(f"{phase}.sandwich_norm(start of a pass)", timed(lambda: LO.sandwich_norm(x, None, None, 1e-5, wf, dtype, add_row=wf)), n * W * (4 + 4 + es), 5.0 * n * W, VECTOR_FLOPS)
+        row(f"{phase}.lokizen.add_rmsnorm", timed(lambda: LO.add_rmsnorm(x, y, None, wn, 1e-5, dtype)), n * W * (4 + 4 + es + es), 4.0 * n * W, VECTOR_FLOPS)
+        # lightning: silu on q, k, v, the recurrence; then norm over all heads and gate  |  Lokizen: retention (rotation, norm per head and gate in its launches)
+        pr = rnd(n, 4 * H * D)
+        cols4 = (0, H * D, 2 * H * D, 3 * H * D)
+        t_li = timed(lambda: LO.linear_scan(pr, cols4[:3], batch, H, H, D, D, state, act=LO.ACT_SILU, decay=decay))
+        row(f"{phase}.linear_scan(lightning)", t_li, n * H * D * (3 * es + 4) + 2 * B * H * D * D * 4, 4.0 * n * H * D * D, VECTOR_FLOPS)
+        raw = torch.randn(n, H * D, device=dev)
+        row(f"{phase}.gated_norm(lightning)", timed(lambda: LO.gated_norm(raw, pr[:, 3 * H * D:], ones, 1e-5, LO.ACT_SIGMOID, False)),
+            n * H * D * (4 + es + es), 8.0 * n * H * D, VECTOR_FLOPS)
+        t_ret = timed(lambda: LO.retention(pr, cols4, batch, H, D, D, D, cos, sin, decay, 1e-5, state))
+        row(f"{phase}.lokizen.retention", t_ret, n * 5 * H * D * es + 2 * B * H * D * D * 4, 4.0 * n * H * D * D, VECTOR_FLOPS)
+        # Mamba-2: convolution (bias, silu), recurrence with decays and steps per token, gate and norm  |  Vumalix: convolution; Mikipel: delta rule
+        mp = rnd(n, H * D + C_ + MH + (-(H * D + C_ + MH)) % 8)
+        cw, cb = rnd(C_, taps), rnd(C_)
+        t_cv = timed(lambda: LO.short_conv(mp, H * D, C_, cw, batch, ctail, LO.ACT_SILU, bias=cb, out_dtype=dtype))
+        row(f"{phase}.short_conv(bias, silu)", t_cv, n * C_ * 2 * es, (2.0 * taps + 5) * n * C_, VECTOR_FLOPS)
+        vw = rnd(W, taps)
+        row(f"{phase}.vumalix.causal_conv", timed(lambda: LO.causal_conv(x, vw, batch, vtail)), n * W * (4 + es), 2.0 * taps * n * W, VECTOR_FLOPS)
+        xbc = LO.short_conv(mp, H * D, C_, cw, batch, ctail, LO.ACT_SILU, bias=cb, out_dtype=dtype)
+        dt = mp[:, H * D + C_:H * D + C_ + MH]
+        t_ma = timed(lambda: LO.linear_scan(xbc, (H * D + MN, H * D, 0), batch, MH, 1, MN, MD, mstate, dt=dt, a_log=a_log, dt_bias=dt_bias, skip=skip))
+        row(f"{phase}.linear_scan(mamba2)", t_ma, n * (C_ * es + MH * es + H * D * 4) + 2 * B * MH * MN * MD * 4, 4.0 * n * MH * MN * MD, VECTOR_FLOPS)
+        row(f"{phase}.gated_norm(mamba2)", timed(lambda: LO.gated_norm(raw, mp[:, :H * D], ones, 1e-5, LO.ACT_SILU, True)),
+            n * H * D * (4 + es + es), 8.0 * n * H * D, VECTOR_FLOPS)
+        qkv = torch.randn(n, 2 * G * D + H * D, device=dev)
+        pd = rnd(n, H * D + 2 * H)
+        t_dl = timed(lambda: LO.delta_rule(qkv, (0, G * D, 2 * G * D), pd, (H * D, H * D + H, 0), da_log, torch.zeros(H, device=dev), dnw, batch, H, G, D, D, 1e-6, D ** -0.5, 1e-6, state))
+        row(f"{phase}.mikipel.delta_rule", t_dl, n * ((2 * G * D + H * D) * 4 + (2 * H * D + 2 * H) * es) + 2 * B * H * D * D * 4, 6.0 * n * H * D * D, VECTOR_FLOPS)
+        # attention: whole-projection norm + rotation + append, then chunked attention with capped scores  |  Lokizen, Bamanex
+        pa = rnd(n, H * D + 2 * G * D + H)
+        cols = (0, H * D, H * D + G * D)
+        wq, wk = rnd(H * D), rnd(G * D)
+        t_qr = timed(lambda: LO.qk_norm_append(pa, cols, H, G, D, D, wq, wk, 1e-5, kc, vc, batch.kv_slot, rot_dims=D // 2, pairing=LO.ROT_NEIGHBOURS, batch=batch, cos=hcos, sin=hsin))
+        row(f"{phase}.qk_norm_append(rot)", t_qr, 2 * n * (H * D + 2 * G * D) * es, 10.0 * n * (H + G) * D, VECTOR_FLOPS)
+        q = LO.qk_norm_append(pa, cols, H, G, D, D, wq, wk, 1e-5, kc, vc, batch.kv_slot)
+        t_qk = timed(lambda: LO.qk_norm_append(pa, cols, H, G, D, D, wq, wk, 1e-5, kc, vc, batch.kv_slot))
+        row(f"{phase}.lokizen.qk_norm_append", t_qk, 2 * n * (H * D + 2 * G * D) * es, 6.0 * n * (H + G) * D, VECTOR_FLOPS)
+        hg = pa[:, H * D + 2 * G * D:]
+        t_at = timed(lambda: LO.attn_sweep(q, kc, vc, batch, H, G, D, D, D ** -0.5, 0, sink=sink, gate=hg, gate_per_head=True, chunk=win, softcap=50.0, out_scale=0.6))
+        row(f"{phase}.attn_chunked(capped)", t_at, span_k * 2 * G * D * es + 2 * n * H * D * es, 4.0 * chunked * H * D, MATRIX_FLOPS)
+        t_bs = timed(lambda: LO.attn_sweep(q, kc, vc, batch, H, G, D, D, D ** -0.5, win, sink=sink, gate=hg, gate_per_head=True))
+        row(f"{phase}.bamanex.attn_sink_gate", t_bs, span_w * 2 * G * D * es + 2 * n * H * D * es, 4.0 * windowed * H * D, MATRIX_FLOPS)
+        gate = rnd(n, H * D)
+        rel, talk = torch.randn(max(prompt_len, context) + 8, H, device=dev), torch.eye(H, device=dev)
+        t_lw = timed(lambda: LO.attn_window(q, gate, kc, vc, batch, H, G, D, D, D ** -0.5, win, 4, rel, None, talk))
+        row(f"{phase}.lokizen.attn_window", t_lw, span_w * 2 * G * D * es + 3 * n * H * D * es, 4.0 * windowed * H * D, MATRIX_FLOPS)
+        gu = rnd(n, 2 * top * ff)
+        row(f"{phase}.gated_act(silu)", timed(lambda: LO.gated_act(gu, 0, top * ff, top * ff, LO.ACT_SILU)), 3 * n * top * ff * es, 6.0 * n * top * ff, VECTOR_FLOPS)
+        row(f"{phase}.qwen2.swiglu", timed(lambda: ops.swiglu(gu)), 3 * n * top * ff * es, 4.0 * n * top * ff, VECTOR_FLOPS)
+    return out
+
+
+def run_safisun(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
+    res = {"bench": "ragged_family", "design": "Safisun", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
+           "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
+    for name in sizes:
+        s = SIZES[name]
+        entry = {"shape": s, "safisun": bench_safisun(s, prompts, prompt_len, decode_batch, context)}
+        torch.cuda.empty_cache()
+        entry["lokizen"] = bench_lokizen(s, prompts, prompt_len, decode_batch, context)
+        torch.cuda.empty_cache()
+        entry["qwen2"] = bench_qwen2(s, prompts, prompt_len, decode_batch, context)
+        torch.cuda.empty_cache()
+        if kernels:
+            entry["kernels"] = kernel_table_safisun(s, prompts, prompt_len, decode_batch, context)
+            torch.cuda.empty_cache()
+        res["sizes"][name] = entry
+    return res
+
+
 def run_mikipel(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
     res = {"bench": "ragged_family", "design": "Mikipel", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
            "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
@@ -594,6 +728,8 @@ def run(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, 
         return run_bamanex(sizes, prompts, prompt_len, decode_batch, context, kernels)
     if design.lower() == "mikipel":
         return run_mikipel(sizes, prompts, prompt_len, decode_batch, context, kernels)
+    if design.lower() == "safisun":
+        return run_safisun(sizes, prompts, prompt_len, decode_batch, context, kernels)
     res = {"bench": "ragged_family", "design": "Lokizen", "closest": "Qwen2", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
            "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
     for name in sizes:
@@ -611,7 +747,7 @@ def run(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, 
 
 def main(argv=None):
     ap = argparse.ArgumentParser(description=__doc__.split("\n")[0])
-    ap.add_argument("--design", default="lokizen", choices=("lokizen", "vumalix", "bamanex", "mikipel"))
+    ap.add_argument("--design", default="lokizen", choices=("lokizen", "vumalix", "bamanex", "mikipel", "safisun"))
     ap.add_argument("--sizes", default="small,medium")
     ap.add_argument("--prompts", type=int, default=4)
     ap.add_argument("--prompt-len", type=int, default=2048)
