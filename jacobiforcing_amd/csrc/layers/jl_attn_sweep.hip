@@ -451,8 +451,17 @@ __global__ __launch_bounds__(AS_THREADS, 2) void attn_rows_kernel(jl_attn_args a
 #pragma unroll
         for (int r = 0; r < 16; ++r) sc[r] *= a.scale;
         if (a.softcap > 0.f) {
+            float big = 0.f;
 #pragma unroll
-            for (int r = 0; r < 16; ++r) sc[r] = soft_cap_fast(sc[r], a.softcap);
+            for (int r = 0; r < 16; ++r) big = fmaxf(big, fabsf(sc[r]));
+            if (__any(big > 0.25f * a.softcap)) {                   // wavefront-uniform: most tiles' scores are far below the cap
+#pragma unroll
+                for (int r = 0; r < 16; ++r) sc[r] = soft_cap_fast(sc[r], a.softcap);
+            } else {
+                const float inv_cap = 1.0f / a.softcap;
+#pragma unroll
+                for (int r = 0; r < 16; ++r) sc[r] = soft_cap_small(sc[r], inv_cap);
+            }
         }
         if (inside) {
 #pragma unroll

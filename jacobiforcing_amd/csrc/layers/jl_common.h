@@ -68,6 +68,11 @@ __device__ __forceinline__ float block_sum_f32(float v, float *red) {
 __device__ __forceinline__ float soft_cap_fast(float s, float cap) {
     return cap - 2.0f * cap * __builtin_amdgcn_rcpf(1.0f + __expf(2.0f * s * __builtin_amdgcn_rcpf(cap)));
 }
+// the same for |s| <= cap / 4 without a transcendental: s (1 - z^2/3 + 2 z^4/15 - 17 z^6/315 + 62 z^8/2835), z = s / cap
+__device__ __forceinline__ float soft_cap_small(float s, float inv_cap) {
+    const float z = s * inv_cap, y = z * z;
+    return s * (1.0f + y * (-0.33333333f + y * (0.13333333f + y * (-0.053968254f + y * 0.021869489f))));
+}
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // gated units of a feed-forward (jl_gated_act, and the grouped product that applies them in its epilogue)
