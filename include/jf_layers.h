@@ -190,8 +190,9 @@ JL_API int jl_causal_conv_carry(const float *x, const int32_t *seq, int32_t B, f
 /* Short causal convolution over time of a column range of a product, with an optional bias and an activation and no residual:
  *   out[t, c] = act(bias[c] + sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start)
  * x [N, ld], w [C, taps] and bias [C] (null: none) of `dtype`, out [N, C] float or of `dtype` (`out_dtype`); act JL_ACT_SILU or JL_ACT_NONE; taps <= 8.  tail float [slots, taps - 1, C] as for
- * jl_causal_conv (the INPUTS at the positions before the step); it is moved on here as well — for requests with one row in the launch
- * itself, for the others (max_count > 1) by a second launch enqueued behind it. */
+ * jl_causal_conv (the INPUTS at the positions before the step); it is moved on here as well — for requests with one row, or from position
+ * 0, in the launch itself, for the others by a second launch enqueued behind it (max_count: the most rows a request with pos0 > 0 has; 1: no
+ * second launch). */
 JL_API int jl_short_conv(const void *x, int dtype, int64_t ld, int32_t col, const void *w, const void *bias, const int32_t *row_req, const int32_t *seq, int32_t B,
                          int32_t max_count, float *tail, int64_t N, int32_t C, int32_t taps, int32_t act, void *out, int out_dtype, void *stream);
 

@@ -143,7 +143,8 @@ extern "C" int jl_causal_conv_carry(const float *x, const int32_t *seq, int32_t 
 //   out[t, c] = act(bias[c] + sum_{j < taps} w[c, j] * x[t - taps + 1 + j, col + c])        (zeros before the sequence's start)
 // A workgroup walks CONV_ROWS consecutive rows, a thread owns VC channels (one, or four with 8- or 16-byte loads) and keeps the last taps - 1
 // inputs in registers.  The tail (float [slots, taps - 1, C]) is read for the inputs before the step and moved on here by requests with
-// ONE row; requests with more rows leave that to short_conv_carry_kernel, enqueued after every row has read.
+// ONE row and by those that start at position 0 (nobody reads their tail); the others leave that to short_conv_carry_kernel, enqueued after
+// every row has read.
 template <int VC, typename P> __device__ __forceinline__ void conv_ld(const P *p, float (&v)[VC]) {
     if constexpr (VC == 4) ld4_f(p, v);
     else v[0] = ld_f(p);
@@ -199,7 +200,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T *__restrict__ x
         for (int s2 = 0; s2 < KEEP; ++s2)
 #pragma unroll
             for (int e = 0; e < VC; ++e) win[s2][e] = s2 + 1 < KEEP ? win[s2 + 1 < KEEP ? s2 + 1 : s2][e] : cur[e];
-        if (count == 1 && KEEP > 0) {
+        if (KEEP > 0 && (count == 1 || (pos0 == 0 && t == count - 1))) {       // the tail's only reader has read it, or it has none
 #pragma unroll
             for (int s2 = 0; s2 < KEEP; ++s2) conv_st<VC>(tail + ((int64_t)slot * KEEP + s2) * C + c, win[s2]);
         }

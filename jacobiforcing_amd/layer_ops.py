@@ -761,8 +761,8 @@ def short_conv(x: torch.Tensor, col: int, C_: int, w: torch.Tensor, batch: Ragge
     _need(bias is None or (bias.dtype == x.dtype and bias.numel() == C_ and bias.is_contiguous()), "short_conv: bias [C] of x's dtype")
     _need(out_dtype in (torch.float32, x.dtype), "short_conv: the output is float or of x's dtype")
     out = torch.empty((n, C_), dtype=out_dtype, device=x.device)
-    N.check_layers(N.layers().jl_short_conv(_ptr(x), _code(x.dtype), ld, col, _ptr(w), _ptr(bias), _ptr(batch.row_req), _ptr(batch.seq), batch.B, max(batch.counts),
-                                           _ptr(tail), n, C_, taps, int(act), _ptr(out), _code(out_dtype), _stream(x.device)), "jl_short_conv")
+    N.check_layers(N.layers().jl_short_conv(_ptr(x), _code(x.dtype), ld, col, _ptr(w), _ptr(bias), _ptr(batch.row_req), _ptr(batch.seq), batch.B,
+                                           max([c for c, s in zip(batch.counts, batch.starts) if s > 0], default=1), _ptr(tail), n, C_, taps, int(act), _ptr(out), _code(out_dtype), _stream(x.device)), "jl_short_conv")
     return out
 
 
