@@ -17,7 +17,7 @@ extern "C" {
 #endif
 
 #define JL_API __attribute__((visibility("default")))
-#define JL_VERSION 125
+#define JL_VERSION 126
 #define JL_OK 0
 #define JL_E_INVALID (-1)
 #define JL_E_LAUNCH (-3)
@@ -28,9 +28,9 @@ JL_API int jl_version(void);
 JL_API const char *jl_last_error(void);
 
 /* x[n, :] = embed[ids[n], :] * scale (float); x0, when given, receives the same rows (the embedding output a repeated pass adds
- * again). */
+ * again); x16, when given, receives them rounded to bfloat16 (a first sublayer that reads the stream itself). */
 JL_API int jl_embed_scale(const void *embed, int dtype, const int64_t *ids, int64_t N, int32_t W, float scale, float *x, float *x0,
-                          void *stream);
+                          void *x16, void *stream);
 
 /* Residual update + RMS norm: x[n] += sum_{s < y_count} y[n * y_count + s] (y of dtype y_dtype, may be null) + x0[n] (float,
  * may be null); then, when `out` is given, out[n] = x[n] / sqrt(mean(x[n]^2) + eps) * w (w of `dtype`, null = no weight). */
@@ -164,6 +164,19 @@ JL_API int jl_norm_add(float *x, const void *y, int y_dtype, const float *g, flo
 JL_API int jl_sandwich_norm(const float *x_in, float *x_out, const void *y, int y_dtype, const float *w_post, const float *add_row, float eps,
                             const float *w_next, void *out, int dtype, int64_t out_ld, int32_t plain, int64_t N, int32_t W, void *stream);
 
+/* Norm on a sublayer's OUTPUT with a weight per channel, residual update, and what the next sublayer reads, in one launch:
+ *   y[n] = sum_a scale_a * sum_{s < count_a} y_a[n, s]                     (at most 3 addends as for jl_scaled_add_norms)
+ *   x[n] += mult * norm(y[n]) * w                                          (no addends: no update)
+ *   out[n] = norm(x[n]) * w_next, or x[n] itself (w_next null), in `dtype`             (out null: the update only)
+ * kind JL_NORM_RMS: norm(v) = v / sqrt(mean(v^2) + eps);  JL_NORM_LAYER: norm(v) = d / sqrt(mean(d^2) + eps) with d = v - mean(v).
+ * With ids / weights [N, top] (a router's choice; null: none), addend 0 holds the experts' outputs, `top` rows per token, and a choice
+ * ids >= n_experts is an identity expert: its row is not read, weights * x[n] (x before the update) stands in for it. */
+#define JL_NORM_RMS 0
+#define JL_NORM_LAYER 1
+JL_API int jl_output_norm(float *x, const jl_addend *addends, int32_t n_addends, const int32_t *ids, const float *weights, int32_t top,
+                          int32_t n_experts, int32_t kind, const float *w, float mult, float eps, const float *w_next, void *out, int dtype,
+                          int64_t N, int32_t W, void *stream);
+
 /* Norm and gate on a recurrent mixer's float output raw [N, C], over `parts` equal parts of the row (each by its own root mean square):
  *   gate_first != 0:  v = raw * act(gate), out = v / sqrt(mean(v^2) + eps) * w * scale
  *   gate_first == 0:  out = raw / sqrt(mean(raw^2) + eps) * w * act(gate) * scale
@@ -221,7 +234,8 @@ JL_API int jl_diff_combine(const float *a1, const float *a2, int64_t ld, int64_t
  *   pool[slot[n]] = [rms_norm(key/value latent) * wkv (R) | rotate(rotary key, pos[n]) (rd)]          (pool rows of R + rd)
  * rotate: of the first rot_dims dimensions, i and i + rot_dims/2 form a pair (u, v) -> (u cos a - v sin a, v cos a + u sin a),
  * a from the cos / sin tables [positions, rot_dims/2] float; the rest pass unchanged (`pairing` JL_ROT_NEIGHBOURS: 2i and 2i + 1 form
- * the pair instead).  Rq = 0: the model has no query latent (wq, cq_out null; nothing is read at q_col). */
+ * the pair instead).  Rq = 0: the model has no query latent (wq, cq_out null; nothing is read at q_col).  pool null: the query latent
+ * alone (a layer that attends over another layer's pool; nothing is read at kv_col). */
 #define JL_ROT_HALVES 0          /* dimension i pairs with i + rot_dims/2 */
 #define JL_ROT_NEIGHBOURS 1      /* dimension 2i pairs with 2i + 1 (angle i) */
 JL_API int jl_latent_prep(const void *proj, int dtype, int64_t N, int64_t ld, int32_t q_col, int32_t Rq, int32_t kv_col, int32_t R,
@@ -300,8 +314,8 @@ JL_API int jl_linear_scan_chunked_ok(int dtype, int32_t D, int32_t Dv);
 /* Router of a mixture of experts over float logits [N, E]; ids [N, top] int32, weights [N, top] float.
  *   JL_ROUTE_SIGMOID:        s = sigmoid(logits); the `top` experts with the largest s + correction are chosen (ties: lowest
  *                            index); weights = s * scale (not renormalised).
- *   JL_ROUTE_SOFTMAX_RENORM: s = softmax(logits) over all experts; the `top` largest are chosen (ties: lowest index); weights =
- *                            s / (sum of the chosen s + renorm_eps) * scale.  `correction` is not read.
+ *   JL_ROUTE_SOFTMAX_RENORM: s = softmax(logits) over all experts; the `top` experts with the largest s + correction (null: s) are chosen
+ *                            (ties: lowest index); weights = s / (sum of the chosen s + renorm_eps) * scale.
  *   JL_ROUTE_TOP_SOFTMAX:    the `top` largest logits are chosen (ties: lowest index); weights = softmax over the chosen logits
  *                            only, times scale.  `correction` is not read. */
 #define JL_ROUTE_SIGMOID 0
@@ -310,7 +324,7 @@ JL_API int jl_linear_scan_chunked_ok(int dtype, int32_t D, int32_t Dv);
 JL_API int jl_moe_route(const float *logits, const float *correction, int64_t N, int32_t E, int32_t top, float scale, int32_t *ids,
                         float *weights, int32_t kind, float renorm_eps, void *stream);
 
-/* Rows (token, choice) grouped by expert.  perm [N*top]: sorted row -> flat index n*top + s; offsets [E+1]; tile_expert /
+/* Rows (token, choice) grouped by expert; a choice outside 0 .. E-1 (an expert without weights) is left out.  perm [N*top]: sorted row -> flat index n*top + s; offsets [E+1]; tile_expert /
  * tile_row0 [max_tiles] (max_tiles >= N*top/tile_rows + E): row tiles of at most tile_rows rows of one expert, unused entries -1. */
 JL_API int jl_moe_group(const int32_t *ids, int64_t N, int32_t top, int32_t E, int32_t tile_rows, int32_t *perm, int32_t *offsets,
                         int32_t *tile_expert, int32_t *tile_row0, int32_t max_tiles, void *stream);

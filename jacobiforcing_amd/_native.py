@@ -231,11 +231,12 @@ def raise_state_error(code: int, what: str, aux: int = 0):
 
 # ---- libjf_layers.so (include/jf_layers.h): layer kernels of the models whose forward is not stock PyTorch ----------------------------
 JL_F32, JL_BF16 = 0, 1
-JL_VERSION = 125                 # include/jf_layers.h: a library of another version is not called (its signatures may differ)
+JL_VERSION = 126                 # include/jf_layers.h: a library of another version is not called (its signatures may differ)
 JL_OUT_SAME, JL_OUT_F32 = 0, 2
 JL_ACT_GELU_TANH, JL_ACT_CLAMPED_SWISH, JL_ACT_SILU, JL_ACT_GELU_ERF, JL_ACT_SIGMOID, JL_ACT_NONE = 0, 1, 2, 3, 4, -1
 JL_ROUTE_SIGMOID, JL_ROUTE_SOFTMAX_RENORM, JL_ROUTE_TOP_SOFTMAX = 0, 1, 2
 JL_ROT_HALVES, JL_ROT_NEIGHBOURS = 0, 1
+JL_NORM_RMS, JL_NORM_LAYER = 0, 1
 JL_MOE_UP_RELU2, JL_MOE_DOWN, JL_MOE_UP_PLAIN = 0, 1, 2
 
 
@@ -264,7 +265,7 @@ class Addend(C.Structure):
 _LAYER_SIGNATURES = {
     "jl_version": (C.c_int, []),
     "jl_last_error": (C.c_char_p, []),
-    "jl_embed_scale": (C.c_int, [_vp, C.c_int, _vp, _i64, _i32, _f32, _vp, _vp, _vp]),
+    "jl_embed_scale": (C.c_int, [_vp, C.c_int, _vp, _i64, _i32, _f32, _vp, _vp, _vp, _vp]),
     "jl_add_rmsnorm": (C.c_int, [_vp, _vp, C.c_int, _i32, _vp, _vp, _f32, _vp, C.c_int, _i64, _i32, _vp]),
     "jl_qk_norm_append": (C.c_int, [_vp, C.c_int, _i64, _i64, _i32, _i32, _i32, _i32, _i32, _i32, _i32, _vp, _vp, _f32, _vp, _vp, _vp, _vp, _i32, _i32,
                                     _vp, _vp, _vp, _vp]),
@@ -293,6 +294,7 @@ _LAYER_SIGNATURES = {
     "jl_softcap": (C.c_int, [_vp, _i64, _f32, _vp]),
     "jl_short_conv": (C.c_int, [_vp, C.c_int, _i64, _i32, _vp, _vp, _vp, _vp, _i32, _i32, _vp, _i64, _i32, _i32, _i32, _vp, C.c_int, _vp]),
     "jl_sandwich_norm": (C.c_int, [_vp, _vp, _vp, C.c_int, _vp, _vp, _f32, _vp, _vp, C.c_int, _i64, _i32, _i64, _i32, _vp]),
+    "jl_output_norm": (C.c_int, [_vp, C.POINTER(Addend), _i32, _vp, _vp, _i32, _i32, _i32, _vp, _f32, _f32, _vp, _vp, C.c_int, _i64, _i32, _vp]),
     "jl_gated_norm": (C.c_int, [_vp, _vp, C.c_int, _i64, _vp, _f32, _i32, _i32, _f32, _vp, _i64, _i64, _i32, _i32, _vp]),
     "jl_linear_scan": (C.c_int, [C.POINTER(ScanArgs), _vp]),
     "jl_linear_scan_chunked_ok": (C.c_int, [C.c_int, _i32, _i32]),

@@ -28,12 +28,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const T *__restrict__ 
     const T *row = proj + n * ld;
     float sq = 0.f, sk = 0.f;
     for (int c = threadIdx.x; c < Rq; c += blockDim.x) { const float v = ld_f(row + q_col + c); sq += v * v; }
-    for (int c = threadIdx.x; c < R; c += blockDim.x) { const float v = ld_f(row + kv_col + c); sk += v * v; }
-    for (int c = threadIdx.x; c < rd; c += blockDim.x) kr[c] = ld_f(row + kv_col + R + c);
+    if (pool) for (int c = threadIdx.x; c < R; c += blockDim.x) { const float v = ld_f(row + kv_col + c); sk += v * v; }
+    if (pool) for (int c = threadIdx.x; c < rd; c += blockDim.x) kr[c] = ld_f(row + kv_col + R + c);
     sq = block_sum_f32(sq, red);
     sk = block_sum_f32(sk, red);                                // its barriers also publish kr
-    const float rq = Rq > 0 ? 1.0f / sqrtf(sq / (float)Rq + eps) : 0.f, rk = 1.0f / sqrtf(sk / (float)R + eps);
+    const float rq = Rq > 0 ? 1.0f / sqrtf(sq / (float)Rq + eps) : 0.f, rk = pool ? 1.0f / sqrtf(sk / (float)R + eps) : 0.f;
     for (int c = threadIdx.x; c < Rq; c += blockDim.x) st_f(cq_out + n * Rq + c, ld_f(row + q_col + c) * rq * ld_f(wq + c));
+    if (!pool) return;
     const int64_t sl = slot[n];
     if (sl < 0) return;
     T *dst = pool + sl * (int64_t)(R + rd);
@@ -47,9 +48,10 @@ extern "C" int jl_latent_prep(const void *proj, int dtype, int64_t N, int64_t ld
                               const float *cos_t, const float *sin_t, int64_t table_len, void *cq_out, void *pool, const int64_t *slot,
                               int32_t pairing, void *stream) {
     if (N <= 0) return JL_OK;
-    if (!proj || !wkv || !pos || !pool || !slot || (Rq > 0 && (!wq || !cq_out))) return jl_fail(JL_E_INVALID, "jl_latent_prep: null pointer");
+    if (!proj || !pos || (pool && (!wkv || !slot)) || (Rq > 0 && (!wq || !cq_out)) || (!pool && Rq <= 0)) return jl_fail(JL_E_INVALID, "jl_latent_prep: null pointer");
+    if (!pool) { R = rd = rot_dims = 0; kv_col = 0; }
     if (pairing != JL_ROT_HALVES && pairing != JL_ROT_NEIGHBOURS) return jl_fail(JL_E_INVALID, "jl_latent_prep: unknown pairing %d", pairing);
-    if (Rq < 0 || R <= 0 || rd < 0 || q_col + (int64_t)Rq > ld || kv_col + (int64_t)R + rd > ld)
+    if (Rq < 0 || (pool && R <= 0) || rd < 0 || q_col + (int64_t)Rq > ld || kv_col + (int64_t)R + rd > ld)
         return jl_fail(JL_E_INVALID, "jl_latent_prep: columns do not fit the row stride");
     if (rot_dims < 0 || rot_dims > rd || (rot_dims & 1) || (rot_dims && (!cos_t || !sin_t || table_len <= 0)))
         return jl_fail(JL_E_INVALID, "jl_latent_prep: rot_dims must be even, at most rd, with angle tables");

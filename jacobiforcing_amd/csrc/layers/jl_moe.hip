@@ -33,19 +33,21 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float *__restrict_
         return;
     }
     if (kind == JL_ROUTE_SOFTMAX_RENORM) {
-        // scores = softmax over ALL experts; the largest `top` (ties: lowest index); weights = score / (sum of the chosen + renorm_eps)
+        // scores = softmax over ALL experts; the largest `top` of score + correction (ties: lowest index); weights = score / (sum of the
+        // chosen scores + renorm_eps).  Without a correction the logits themselves are compared.
         float zmax = -INFINITY, den = 0.f, chosen = 0.f;
         for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
         for (int e = 0; e < E; ++e) den += expf(z[e] - zmax);
         for (int s = 0; s < top; ++s) {
             int best = -1;
-            float bz = 0.f;
+            float bc = 0.f;
             for (int e = 0; e < E; ++e) {
                 bool taken = false;
                 for (int p = 0; p < s; ++p) taken |= ids[n * top + p] == e;
-                if (!taken && (best < 0 || z[e] > bz)) { best = e; bz = z[e]; }
+                const float ch = correction ? expf(z[e] - zmax) / den + correction[e] : z[e];
+                if (!taken && (best < 0 || ch > bc)) { best = e; bc = ch; }
             }
-            const float sc = expf(bz - zmax) / den;
+            const float sc = expf(z[best] - zmax) / den;
             ids[n * top + s] = best;
             weights[n * top + s] = sc;
             chosen += sc;
@@ -92,7 +94,10 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restri
     __shared__ int base[MOE_MAX_E + 1];
     for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
     __syncthreads();
-    for (int64_t r = threadIdx.x; r < rows; r += 1024) atomicAdd(&cnt[ids[r]], 1);
+    for (int64_t r = threadIdx.x; r < rows; r += 1024) {
+        const int e = ids[r];
+        if (e >= 0 && e < E) atomicAdd(&cnt[e], 1);                   // an expert without weights has no rows
+    }
     __syncthreads();
     if (threadIdx.x == 0) {
         int o = 0, t = 0;
@@ -113,7 +118,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restri
     __syncthreads();
     for (int64_t r = threadIdx.x; r < rows; r += 1024) {
         const int e = ids[r];
-        perm[base[e] + atomicAdd(&cnt[e], 1)] = (int32_t)r;
+        if (e >= 0 && e < E) perm[base[e] + atomicAdd(&cnt[e], 1)] = (int32_t)r;
     }
 }
 

@@ -4,21 +4,22 @@
 
 template <typename T>
 __global__ __launch_bounds__(256) void embed_scale_kernel(const T *__restrict__ embed, const int64_t *__restrict__ ids, int W,
-                                                           float scale, float *__restrict__ x, float *__restrict__ x0) {
+                                                           float scale, float *__restrict__ x, float *__restrict__ x0, bf16_t *__restrict__ x16) {
     const int64_t n = blockIdx.x;
     const T *src = embed + ids[n] * (int64_t)W;
     for (int c = threadIdx.x; c < W; c += 256) {
         const float v = ld_f(src + c) * scale;
         x[n * W + c] = v;
         if (x0) x0[n * W + c] = v;
+        if (x16) st_f(x16 + n * W + c, v);
     }
 }
 
 extern "C" int jl_embed_scale(const void *embed, int dtype, const int64_t *ids, int64_t N, int32_t W, float scale, float *x, float *x0,
-                              void *stream) {
+                              void *x16, void *stream) {
     if (N <= 0) return JL_OK;
     if (!embed || !ids || !x || W <= 0) return jl_fail(JL_E_INVALID, "jl_embed_scale: null pointer or bad width");
-    JL_DISPATCH(dtype, embed_scale_kernel<T><<<dim3((unsigned)N), 256, 0, (hipStream_t)stream>>>((const T *)embed, ids, W, scale, x, x0));
+    JL_DISPATCH(dtype, embed_scale_kernel<T><<<dim3((unsigned)N), 256, 0, (hipStream_t)stream>>>((const T *)embed, ids, W, scale, x, x0, (bf16_t *)x16));
     return jl_check_launch("embed_scale_kernel");
 }
 
@@ -587,6 +588,186 @@ extern "C" int jl_sandwich_norm(const float *x_in, float *x_out, const void *y, 
 #undef SN_CASE
 #undef SN_ARGS
     return jl_check_launch("sandwich_norm_kernel");
+}
+
+// ---- norm on a sublayer's output (RMS or layer norm), residual update, and what the next sublayer reads -----------------------------------
+// The sublayer's output y is the sum of up to three addends; the routed experts' addend (the first, `top` rows per token) reads no row where
+// the choice is an identity expert (ids >= n_experts): its contribution is weight * x.  One workgroup per row.  The vector form keeps y and x
+// in registers from the first load to the last store; the variance is the mean of the squared deviations from a mean formed before.
+struct OutNormArgs {
+    float *x; jl_addend ad[3]; const int32_t *ids; const float *weights; const float *w; const float *w_next; void *out;
+    int32_t top, n_experts, kind, W;
+    float mult, eps;
+};
+
+__device__ __forceinline__ float out_norm_y(const OutNormArgs &a, int64_t n, int c) {
+    float y = 0.f;
+#pragma unroll
+    for (int k = 0; k < 3; ++k) {
+        if (!a.ad[k].y) continue;
+        float u = 0.f;
+        for (int s = 0; s < a.ad[k].count; ++s) {
+            if (k == 0 && a.ids && a.ids[n * a.top + s] >= a.n_experts) u += a.weights[n * a.top + s] * a.x[n * a.W + c];
+            else u += ld_any(a.ad[k].y, a.ad[k].dtype, (n * a.ad[k].count + s) * (int64_t)a.W + c);
+        }
+        y += a.ad[k].scale ? u * a.ad[k].scale[c] : u;
+    }
+    return y;
+}
+
+// any width: y is formed anew for the mean, the deviations and the update; x of a channel is read and written by one thread only
+template <typename T>
+__global__ __launch_bounds__(256) void output_norm_kernel(OutNormArgs a) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int W = a.W;
+    float *xr = a.x + n * W;
+    const bool update = a.ad[0].y || a.ad[1].y || a.ad[2].y;
+    float mean = 0.f;
+    if (update) {
+        if (a.kind == JL_NORM_LAYER) {
+            float s = 0.f;
+            for (int c = threadIdx.x; c < W; c += 256) s += out_norm_y(a, n, c);
+            mean = block_sum_f32(s, red) / (float)W;
+        }
+        float ss = 0.f;
+        for (int c = threadIdx.x; c < W; c += 256) { const float d = out_norm_y(a, n, c) - mean; ss += d * d; }
+        const float r = a.mult / sqrtf(block_sum_f32(ss, red) / (float)W + a.eps);
+        for (int c = threadIdx.x; c < W; c += 256) xr[c] += (out_norm_y(a, n, c) - mean) * r * a.w[c];
+    }
+    if (!a.out) return;
+    T *o = (T *)a.out + n * W;
+    if (!a.w_next) {
+        for (int c = threadIdx.x; c < W; c += 256) st_f(o + c, xr[c]);
+        return;
+    }
+    mean = 0.f;
+    if (a.kind == JL_NORM_LAYER) {
+        float s = 0.f;
+        for (int c = threadIdx.x; c < W; c += 256) s += xr[c];
+        mean = block_sum_f32(s, red) / (float)W;
+    }
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < W; c += 256) { const float d = xr[c] - mean; ss += d * d; }
+    const float r = 1.0f / sqrtf(block_sum_f32(ss, red) / (float)W + a.eps);
+    for (int c = threadIdx.x; c < W; c += 256) st_f(o + c, (xr[c] - mean) * r * a.w_next[c]);
+}
+
+// v (VI groups of four channels per thread) -> v - mean (layer norm), and 1 / sqrt(mean square + eps) of what is left
+template <int VI>
+__device__ __forceinline__ float centre_and_scale(float (&v)[VI][4], int W, int kind, float eps, float *red) {
+    const int step = blockDim.x * 4;
+    if (kind == JL_NORM_LAYER) {
+        float s = 0.f;
+#pragma unroll
+        for (int i = 0; i < VI; ++i)
+            if (i * step + (int)threadIdx.x * 4 < W) s += v[i][0] + v[i][1] + v[i][2] + v[i][3];
+        const float mean = block_sum_f32(s, red) / (float)W;
+#pragma unroll
+        for (int i = 0; i < VI; ++i)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[i][e] -= mean;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < VI; ++i)
+        if (i * step + (int)threadIdx.x * 4 < W) ss += v[i][0] * v[i][0] + v[i][1] * v[i][1] + v[i][2] * v[i][2] + v[i][3] * v[i][3];
+    return 1.0f / sqrtf(block_sum_f32(ss, red) / (float)W + eps);
+}
+
+template <typename T, int VI>
+__global__ __launch_bounds__(256) void output_norm_vec_kernel(OutNormArgs a) {
+    __shared__ float red[16];
+    const int64_t n = blockIdx.x;
+    const int W = a.W, step = blockDim.x * 4;
+    float x[VI][4], y[VI][4];
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x[i][e] = y[i][e] = 0.f;
+        if (c < W) ld4_f(a.x + n * W + c, x[i]);
+    }
+    if (a.ad[0].y || a.ad[1].y || a.ad[2].y) {
+#pragma unroll
+        for (int k = 0; k < 3; ++k) {
+            if (!a.ad[k].y) continue;
+            float u[VI][4] = {};
+            for (int s = 0; s < a.ad[k].count; ++s) {
+                const bool self = k == 0 && a.ids && a.ids[n * a.top + s] >= a.n_experts;
+                const float ws = self ? a.weights[n * a.top + s] : 0.f;
+#pragma unroll
+                for (int i = 0; i < VI; ++i) {
+                    const int c = i * step + threadIdx.x * 4;
+                    if (c >= W) continue;
+                    float t[4];
+                    if (!self) ld4_any(a.ad[k].y, a.ad[k].dtype, (n * a.ad[k].count + s) * (int64_t)W + c, t);
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) u[i][e] += self ? ws * x[i][e] : t[e];
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < VI; ++i) {
+                const int c = i * step + threadIdx.x * 4;
+                if (c >= W) continue;
+                float sc[4] = {1.f, 1.f, 1.f, 1.f};
+                if (a.ad[k].scale) ld4_f(a.ad[k].scale + c, sc);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[i][e] += u[i][e] * sc[e];
+            }
+        }
+        const float r = a.mult * centre_and_scale<VI>(y, W, a.kind, a.eps, red);
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int c = i * step + threadIdx.x * 4;
+            if (c >= W) continue;
+            float g[4];
+            ld4_f(a.w + c, g);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[i][e] += y[i][e] * r * g[e];
+            st4_f(a.x + n * W + c, x[i]);
+        }
+    }
+    if (!a.out) return;
+    float r = 1.0f;
+    if (a.w_next) r = centre_and_scale<VI>(x, W, a.kind, a.eps, red);
+#pragma unroll
+    for (int i = 0; i < VI; ++i) {
+        const int c = i * step + threadIdx.x * 4;
+        if (c >= W) continue;
+        float g[4] = {1.f, 1.f, 1.f, 1.f};
+        if (a.w_next) ld4_f(a.w_next + c, g);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) g[e] *= x[i][e] * r;
+        st4_f((T *)a.out + n * W + c, g);
+    }
+}
+
+extern "C" int jl_output_norm(float *x, const jl_addend *addends, int32_t n_addends, const int32_t *ids, const float *weights, int32_t top, int32_t n_experts,
+                              int32_t kind, const float *w, float mult, float eps, const float *w_next, void *out, int dtype, int64_t N, int32_t W, void *stream) {
+    if (N <= 0) return JL_OK;
+    if (!x || W <= 0 || n_addends < 0 || n_addends > 3 || (n_addends && (!addends || !w)))
+        return jl_fail(JL_E_INVALID, "jl_output_norm: null pointer, bad width or more than 3 addends");
+    if (kind != JL_NORM_RMS && kind != JL_NORM_LAYER) return jl_fail(JL_E_INVALID, "jl_output_norm: unknown norm %d", kind);
+    OutNormArgs a = {x, {{nullptr, 0, 0, nullptr}, {nullptr, 0, 0, nullptr}, {nullptr, 0, 0, nullptr}}, ids, weights, w, w_next, out, top, n_experts, kind, W, mult, eps};
+    for (int k = 0; k < n_addends; ++k) {
+        a.ad[k] = addends[k];
+        if (!a.ad[k].y || a.ad[k].count <= 0) return jl_fail(JL_E_INVALID, "jl_output_norm: addend %d is null or has no rows", k);
+    }
+    if (ids && (!weights || n_addends < 1 || top != a.ad[0].count || n_experts < 0))
+        return jl_fail(JL_E_INVALID, "jl_output_norm: identity choices go with weights and a first addend of `top` rows per token");
+    auto al = [](const void *q, uintptr_t b) { return ((uintptr_t)q % b) == 0; };
+    bool vec = W % 4 == 0 && W <= 8192 && al(x, 16) && al(w, 16) && al(w_next, 16) && al(out, dtype == JL_BF16 ? 8 : 16);
+    for (int k = 0; k < n_addends; ++k) vec = vec && al(a.ad[k].y, a.ad[k].dtype == JL_BF16 ? 8 : 16) && al(a.ad[k].scale, 16);
+    hipStream_t st = (hipStream_t)stream;
+    const dim3 grid((unsigned)N);
+    const int threads = W >= 1024 ? 256 : (W / 4 + 63) / 64 * 64;
+    if (!vec) JL_DISPATCH(dtype, output_norm_kernel<T><<<grid, 256, 0, st>>>(a));
+    else if (W <= 1024) JL_DISPATCH(dtype, (output_norm_vec_kernel<T, 1><<<grid, threads, 0, st>>>(a)));
+    else if (W <= 2048) JL_DISPATCH(dtype, (output_norm_vec_kernel<T, 2><<<grid, threads, 0, st>>>(a)));
+    else if (W <= 4096) JL_DISPATCH(dtype, (output_norm_vec_kernel<T, 4><<<grid, threads, 0, st>>>(a)));
+    else JL_DISPATCH(dtype, (output_norm_vec_kernel<T, 8><<<grid, threads, 0, st>>>(a)));
+    return jl_check_launch("output_norm_kernel");
 }
 
 // ---- norm over equal parts of a mixer's output with its gate: one workgroup per (row, part) -------------------------------------------------

@@ -147,17 +147,20 @@ class RaggedBatch:
 
 
 def embed_scale(embed: torch.Tensor, ids: torch.Tensor, scale: float, want_copy: bool,
-                out: Optional[torch.Tensor] = None) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
-    """Rows ``ids`` of ``embed`` times ``scale`` as float [N, W] (written into ``out`` when given), and a second copy with ``want_copy``."""
+                out: Optional[torch.Tensor] = None, copy_dtype: torch.dtype = torch.float32) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """Rows ``ids`` of ``embed`` times ``scale`` as float [N, W] (written into ``out`` when given), and a second copy with ``want_copy``
+    (float, or rounded to bfloat16 with ``copy_dtype``)."""
     _dev(embed)
     _need(embed.dim() == 2 and embed.is_contiguous() and ids.dtype == torch.int64 and ids.is_contiguous(), "embed_scale: embed [V, W], ids int64 [N]")
     n, W = ids.numel(), embed.shape[1]
     if out is not None:
         _need(out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (n, W), "embed_scale: out float [N, W]")
     x = out if out is not None else torch.empty((n, W), dtype=torch.float32, device=embed.device)
-    x0 = torch.empty_like(x) if want_copy else None
-    N.check_layers(N.layers().jl_embed_scale(_ptr(embed), _code(embed.dtype), _ptr(ids), n, W, float(scale), _ptr(x), _ptr(x0),
-                                            _stream(embed.device)), "jl_embed_scale")
+    _need(copy_dtype in (torch.float32, torch.bfloat16), "embed_scale: the copy is float or bfloat16")
+    x0 = torch.empty((n, W), dtype=copy_dtype, device=embed.device) if want_copy else None
+    wide = copy_dtype == torch.float32
+    N.check_layers(N.layers().jl_embed_scale(_ptr(embed), _code(embed.dtype), _ptr(ids), n, W, float(scale), _ptr(x), _ptr(x0) if wide else None,
+                                            None if wide else _ptr(x0), _stream(embed.device)), "jl_embed_scale")
     return x, x0
 
 
@@ -380,31 +383,35 @@ _ROUTES = {"sigmoid": N.JL_ROUTE_SIGMOID, "softmax_renorm": N.JL_ROUTE_SOFTMAX_R
 
 def moe_experts(h: torch.Tensor, router_logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, scale: float,
                 w_up: torch.Tensor, w_down: torch.Tensor, route: str = "sigmoid", renorm_eps: float = 0.0,
-                gated: Optional[Tuple[int, float, float, float]] = None) -> torch.Tensor:
+                gated: Optional[Tuple[int, float, float, float]] = None, identity: int = 0):
     """Routed experts: h [N, W], router_logits float [N, E], w_down [E, W, ff].  Returns the weighted expert outputs per choice,
     float [N, top, W] (their sum over the middle axis is the layer's output).
 
     ``route`` "sigmoid": sigmoid scores, choice by score + correction, weights = score * scale; "softmax_renorm": softmax over all
-    experts, the largest chosen, weights = score / (sum of the chosen + renorm_eps) * scale; "top_softmax": the largest logits chosen,
+    experts, the largest score + correction chosen, weights = score / (sum of the chosen scores + renorm_eps) * scale; "top_softmax": the largest logits chosen,
     weights = softmax over the chosen logits only, times scale.
     ``gated`` None: experts down(relu(up h)^2) with w_up [E, ff, W].  ``gated`` = (kind, limit, alpha, shift) of ``gated_act``: w_up
-    [E, 2*ff, W] stacks every expert's gate rows on its linear rows, and the up product applies the unit in its epilogue."""
+    [E, 2*ff, W] stacks every expert's gate rows on its linear rows, and the up product applies the unit in its epilogue.
+    ``identity``: so many router outputs behind the E experts are identity experts, which have no weights and hand their input through.  Then
+    returns (outputs, choice ids int32 [N, top], weights float [N, top]); the rows of outputs whose id is >= E are NOT written — what adds
+    the outputs up (``output_norm``) puts weight * input in their place."""
     _dev(h)
     n, W = h.shape
     E, ff = w_down.shape[0], w_down.shape[2]
+    Er = E + identity
     up_rows = 2 * ff if gated is not None else ff
     dev, dt = h.device, h.dtype
-    _need(h.is_contiguous() and router_logits.dtype == torch.float32 and router_logits.is_contiguous() and tuple(router_logits.shape) == (n, E),
-          "moe_experts: h [N, W], logits float [N, E]")
+    _need(h.is_contiguous() and router_logits.dtype == torch.float32 and router_logits.is_contiguous() and tuple(router_logits.shape) == (n, Er) and identity >= 0,
+          "moe_experts: h [N, W], logits float [N, experts + identity experts]")
     _need(tuple(w_up.shape) == (E, up_rows, W) and tuple(w_down.shape) == (E, W, ff) and w_up.dtype == dt and w_down.dtype == dt and
           w_up.is_contiguous() and w_down.is_contiguous(), "moe_experts: expert weights [E, ff (2*ff when gated), W] / [E, W, ff] in the activation dtype")
-    _need(route in _ROUTES and 1 <= top <= E, "moe_experts: route is 'sigmoid', 'softmax_renorm' or 'top_softmax', 1 <= top <= experts")
+    _need(route in _ROUTES and 1 <= top <= Er, "moe_experts: route is 'sigmoid', 'softmax_renorm' or 'top_softmax', 1 <= top <= experts")
     if correction is not None:
-        _need(correction.dtype == torch.float32 and correction.numel() == E, "moe_experts: correction float [E]")
+        _need(correction.dtype == torch.float32 and correction.numel() == Er, "moe_experts: correction float, one per router output")
     L, st = N.layers(), _stream(dev)
     ids = torch.empty((n, top), dtype=torch.int32, device=dev)
     wts = torch.empty((n, top), dtype=torch.float32, device=dev)
-    N.check_layers(L.jl_moe_route(_ptr(router_logits), _ptr(correction), n, E, top, float(scale), _ptr(ids), _ptr(wts),
+    N.check_layers(L.jl_moe_route(_ptr(router_logits), _ptr(correction), n, Er, top, float(scale), _ptr(ids), _ptr(wts),
                                   _ROUTES[route], float(renorm_eps), st), "jl_moe_route")
     tm = int(L.jl_moe_tile_rows())
     rows = n * top
@@ -427,7 +434,7 @@ def moe_experts(h: torch.Tensor, router_logits: torch.Tensor, correction: Option
     y = torch.empty((n, top, W), dtype=torch.float32, device=dev)
     N.check_layers(L.jl_moe_gemm(_ptr(act), _ptr(w_down), _code(dt), N.JL_MOE_DOWN, ff, W, top, _ptr(perm), _ptr(offsets), _ptr(tile_e), _ptr(tile_r), max_tiles,
                                  _ptr(wts), _ptr(y), st), "jl_moe_gemm(down)")
-    return y
+    return (y, ids, wts) if identity else y
 
 
 ACT_GELU_TANH, ACT_CLAMPED_SWISH, ACT_SILU, ACT_GELU_ERF = N.JL_ACT_GELU_TANH, N.JL_ACT_CLAMPED_SWISH, N.JL_ACT_SILU, N.JL_ACT_GELU_ERF
@@ -494,6 +501,37 @@ def norm_add(x: torch.Tensor, y: torch.Tensor, g: torch.Tensor, eps: float, out_
     out = torch.empty((n, W), dtype=out_dtype, device=x.device) if out_dtype is not None else None
     N.check_layers(N.layers().jl_norm_add(_ptr(x), _ptr(y), _code(y.dtype), _ptr(g), float(eps), _ptr(out), _code(out_dtype or torch.float32), n, W,
                                          _stream(x.device)), "jl_norm_add")
+    return out
+
+
+NORM_RMS, NORM_LAYER = N.JL_NORM_RMS, N.JL_NORM_LAYER
+
+
+def output_norm(x: torch.Tensor, addends: Sequence[Tuple[torch.Tensor, Optional[torch.Tensor]]], w: Optional[torch.Tensor], eps: float, kind: int, mult: float = 1.0,
+                w_next: Optional[torch.Tensor] = None, out_dtype: Optional[torch.dtype] = None,
+                choices: Optional[Tuple[torch.Tensor, torch.Tensor, int]] = None) -> Optional[torch.Tensor]:
+    """x (float [N, W], in place) += mult * norm(sum of the addends) * w — a norm on a sublayer's OUTPUT, RMS (``NORM_RMS``) or layer norm
+    (``NORM_LAYER``), w float [W]; addends (y [N, W] or [N, S, W], channel scale or None), at most three, none: no update.  Returns, in
+    ``out_dtype`` (None: nothing), norm(x) * w_next, or x itself without ``w_next``.
+    ``choices`` = (ids, weights, E): the first addend is what ``moe_experts`` returned with identity experts; choices >= E stand for
+    weight * x (x before the update)."""
+    _dev(x)
+    n, W = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous() and len(addends) <= 3, "output_norm: x contiguous float32 [N, W], at most 3 addends")
+    arr = _addends(addends, n, W, "output_norm")
+    for v in (w, w_next):
+        _need(v is None or (v.dtype == torch.float32 and v.numel() == W and v.is_contiguous()), "output_norm: weights are float [W]")
+    _need(w is not None or not addends, "output_norm: an update needs the norm's weight")
+    ids = wts = None
+    top = E = 0
+    if choices is not None:
+        ids, wts, E = choices
+        _need(len(addends) >= 1 and addends[0][0].dim() == 3 and tuple(ids.shape) == tuple(wts.shape) == tuple(addends[0][0].shape[:2]) and ids.dtype == torch.int32 and
+              wts.dtype == torch.float32 and ids.is_contiguous() and wts.is_contiguous(), "output_norm: choices int32 / float [N, top] of the first addend [N, top, W]")
+        top = ids.shape[1]
+    out = torch.empty((n, W), dtype=out_dtype, device=x.device) if out_dtype is not None else None
+    N.check_layers(N.layers().jl_output_norm(_ptr(x), arr, len(addends), _ptr(ids), _ptr(wts), top, int(E), int(kind), _ptr(w), float(mult), float(eps), _ptr(w_next),
+                                            _ptr(out), _code(out_dtype or torch.float32), n, W, _stream(x.device)), "jl_output_norm")
     return out
 
 
@@ -622,16 +660,20 @@ def _angle_tables(rot_dims: int, cos, sin, batch: RaggedBatch, what: str) -> int
 ROT_HALVES, ROT_NEIGHBOURS = N.JL_ROT_HALVES, N.JL_ROT_NEIGHBOURS      # which dimensions a rotation pairs: i with i + dims/2, or 2i with 2i + 1
 
 
-def latent_prep(proj: torch.Tensor, q_col: int, Rq: int, kv_col: int, R: int, rd: int, rot_dims: int, wq: Optional[torch.Tensor], wkv: torch.Tensor,
-                eps: float, batch: RaggedBatch, cos, sin, pool: torch.Tensor, pairing: int = N.JL_ROT_HALVES) -> Optional[torch.Tensor]:
+def latent_prep(proj: torch.Tensor, q_col: int, Rq: int, kv_col: int, R: int, rd: int, rot_dims: int, wq: Optional[torch.Tensor], wkv: Optional[torch.Tensor],
+                eps: float, batch: RaggedBatch, cos, sin, pool: Optional[torch.Tensor], pairing: int = N.JL_ROT_HALVES) -> Optional[torch.Tensor]:
     """Normalised query latent [N, Rq] (None with Rq = 0: a model without one); the pool row of every token becomes [normalised key/value
-    latent | rotated shared key]."""
+    latent | rotated shared key].  ``pool`` None: the query latent alone (a layer that attends over another layer's pool)."""
     _dev(proj)
     n, ld = proj.shape
     dt = proj.dtype
-    _need(proj.is_contiguous() and n == batch.N and (Rq == 0 or (wq is not None and wq.numel() == Rq and wq.dtype == dt)) and wkv.numel() == R and wkv.dtype == dt,
+    _need(proj.is_contiguous() and n == batch.N and (Rq == 0 or (wq is not None and wq.numel() == Rq and wq.dtype == dt)) and
+          (pool is None or (wkv is not None and wkv.numel() == R and wkv.dtype == dt)),
           "latent_prep: proj [N, ld] of the batch, norm weights over the latents")
-    _need(pool.dtype == dt and pool.is_contiguous() and pool.shape[-1] == R + rd, "latent_prep: pool [tokens, R + rd]")
+    _need(pool is None or (pool.dtype == dt and pool.is_contiguous() and pool.shape[-1] == R + rd), "latent_prep: pool [tokens, R + rd]")
+    _need(pool is not None or Rq > 0, "latent_prep: neither a query latent nor a pool")
+    if pool is None:
+        R = rd = rot_dims = 0
     tl = _angle_tables(rot_dims, cos, sin, batch, "latent_prep")
     cq = torch.empty((n, Rq), dtype=dt, device=proj.device) if Rq else None
     N.check_layers(N.layers().jl_latent_prep(_ptr(proj), _code(dt), n, ld, q_col, Rq, kv_col, R, rd, rot_dims, _ptr(wq) if Rq else None, _ptr(wkv), float(eps),
@@ -653,6 +695,40 @@ def latent_q_pack(qa: torch.Tensor, q: torch.Tensor, H: int, D: int, R: int, rd:
     N.check_layers(N.layers().jl_latent_q_pack(_ptr(qa), _ptr(q), q.stride(0), _code(q.dtype), n, H, D, R, rd, rot_dims, _ptr(batch.pos), _ptr(cos), _ptr(sin), tl,
                                               _ptr(out), int(pairing), _stream(q.device)), "jl_latent_q_pack")
     return out
+
+
+def latent_attend(qf: torch.Tensor, pool: torch.Tensor, w_uv: torch.Tensor, batch: RaggedBatch, H: int, R: int, rd: int, scale: float, window: int,
+                  sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Latent attention over the pool and the value up-projection behind it: qf [N, H*(R + rd)] (``latent_q_pack``), pool [tokens, R + rd]
+    whose first R columns are the values, w_uv [H, R, Dv] -> [H, N, Dv].  ``window`` 0: plain causal; ``sink`` float [H]; ``gate`` [N, H] view:
+    one sigmoid gate per head on its output (applied to the latent output: the up-projection is linear).  The launch is chosen by dtype and
+    sizes; what no launch takes at once goes in column ranges of the latent, then in groups of heads."""
+    n, W, dt = qf.shape[0], R + rd, qf.dtype
+    per_head = gate is not None
+    up = lambda o, c0, c1, h0, h1: (o.view(n, h1 - h0, c1 - c0).transpose(0, 1), w_uv[h0:h1] if c1 - c0 == R else w_uv[h0:h1, c0:c1].contiguous())
+    if attn_sweep_tile_rows(dt, H, 1, W, R, pool, pool[:, :R]):                    # bfloat16, latents in multiples of 32 up to 512
+        o = attn_sweep(qf, pool, pool[:, :R], batch, H, 1, W, R, scale, window, sink=sink, gate=gate, gate_per_head=per_head)
+        return torch.bmm(*up(o, 0, R, 0, H))
+    fits = lambda h, c: int(N.layers().jl_attn_tile_rows(_code(dt), h, 1, W, c, pool.stride(0), pool.stride(0))) > 0
+    heads, step = H, min(R, ATTN_MAX_VALUE_WIDTH) if dt == torch.bfloat16 else R   # bfloat16: the matrix-core kernel's value tile
+    while not fits(heads, step) and (heads > 1 or step > 8):                       # columns in multiples of eight: the ranges stay aligned
+        if step > 16 or heads == 1:
+            step = (step // 2 + 7) // 8 * 8
+        else:
+            heads, step = -(-heads // 2), min(R, ATTN_MAX_VALUE_WIDTH)
+    parts = []
+    for h0 in range(0, H, heads):
+        h1 = min(H, h0 + heads)
+        q = qf if h1 - h0 == H else qf[:, h0 * W:h1 * W].contiguous()
+        s_, g_ = sink[h0:h1].contiguous() if sink is not None else None, gate[:, h0:h1] if gate is not None else None
+        ov = None
+        for c0 in range(0, R, step):
+            c1 = min(R, c0 + step)
+            o = attn_window(q, g_, pool, pool[:, c0:c1], batch, h1 - h0, 1, W, c1 - c0, scale, window, 0, None, None, None, sink=s_, gate_per_head=per_head)
+            o, wv = up(o, c0, c1, h0, h1)
+            ov = torch.bmm(o, wv) if ov is None else torch.baddbmm(ov, o, wv)
+        parts.append(ov)
+    return parts[0] if len(parts) == 1 else torch.cat(parts, 0)
 
 
 def heads_gate(ov: torch.Tensor, gate: Optional[torch.Tensor]) -> torch.Tensor:

@@ -17,6 +17,7 @@ MODEL_REGISTRY = {
     "Bamanex": ("jacobiforcing_amd.modeling.bamanex", "BamanexConfig", "ragged"),
     "Mikipel": ("jacobiforcing_amd.modeling.mikipel", "MikipelConfig", "ragged"),
     "Safisun": ("jacobiforcing_amd.modeling.safisun", "SafisunConfig", "ragged"),
+    "Voborax": ("jacobiforcing_amd.modeling.voborax", "VoboraxConfig", "ragged"),
 }
 
 
@@ -32,6 +33,20 @@ def read_model_config(model_dir):
         raise ValueError(f"{model_dir}: architecture {arch!r} is not served (known: {sorted(MODEL_REGISTRY)})")
     mod, cls, _ = MODEL_REGISTRY[arch]
     return getattr(importlib.import_module(mod), cls).from_json(Path(model_dir) / "config.json")
+
+
+def read_tensors(model_dir):
+    """Every tensor of the directory's *.safetensors by name, on the host."""
+    from safetensors import safe_open
+    files = sorted(Path(model_dir).glob("*.safetensors"))
+    if not files:
+        raise FileNotFoundError(f"no *.safetensors under {model_dir}")
+    tensors = {}
+    for f in files:
+        with safe_open(str(f), "pt", "cpu") as sf:
+            for k in sf.keys():
+                tensors[k] = sf.get_tensor(k)
+    return tensors
 
 
 def family_of(hf_config) -> str:

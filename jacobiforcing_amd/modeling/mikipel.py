@@ -28,6 +28,7 @@ from typing import Any, Dict, List, Optional
 import torch
 import torch.nn.functional as F
 
+from . import read_tensors
 from .. import layer_ops as LO
 from ..engine.state_cache import PagedStateCache, RunSpec
 
@@ -161,16 +162,7 @@ class MikipelWeights:
 
     @classmethod
     def from_safetensors(cls, cfg: MikipelConfig, model_dir, device, dtype=torch.bfloat16) -> "MikipelWeights":
-        from safetensors import safe_open
-        files = sorted(Path(model_dir).glob("*.safetensors"))
-        if not files:
-            raise FileNotFoundError(f"no *.safetensors under {model_dir}")
-        tensors = {}
-        for f in files:
-            with safe_open(str(f), "pt", "cpu") as sf:
-                for k in sf.keys():
-                    tensors[k] = sf.get_tensor(k)
-        return cls(cfg, tensors, device, dtype)
+        return cls(cfg, read_tensors(model_dir), device, dtype)
 
     @classmethod
     def random(cls, cfg: MikipelConfig, device, dtype=torch.bfloat16, seed: int = 0) -> "MikipelWeights":
@@ -287,21 +279,7 @@ class MikipelModel:
         q = proj[:, :H * (D + rd)]
         qa = torch.bmm(q.view(n, H, D + rd)[:, :, :D].transpose(0, 1), w["w_uk"])                  # [H, N, R]: query . (W_uk c) = (W_uk^T query) . c
         qf = LO.latent_q_pack(qa, q, H, D, R, rd, dims, batch, cos, sin, pairing=LO.ROT_NEIGHBOURS)
-        step = LO.ATTN_MAX_VALUE_WIDTH
-        if LO.attn_sweep_tile_rows(self.dtype, H, 1, R + rd, R, pool, pool[:, :R]):                 # bfloat16, latents in multiples of 32 up to 512
-            o = LO.attn_sweep(qf, pool, pool[:, :R], batch, H, 1, R + rd, R, scale, 0)
-            ov = torch.bmm(o.view(n, H, R).transpose(0, 1), w["w_uv"])
-        elif R <= step or self.dtype != torch.bfloat16:
-            o = LO.attn_window(qf, None, pool, pool[:, :R], batch, H, 1, R + rd, R, scale, 0, 0, None, None, None)
-            ov = torch.bmm(o.view(n, H, R).transpose(0, 1), w["w_uv"])                               # [H, N, Dv]
-        else:           # a latent wider than the matrix-core kernel's value tile: a launch per column range of the latent
-            ov = None
-            for c0 in range(0, R, step):
-                c1 = min(R, c0 + step)
-                o = LO.attn_window(qf, None, pool, pool[:, c0:c1], batch, H, 1, R + rd, c1 - c0, scale, 0, 0, None, None, None)
-                o = o.view(n, H, c1 - c0).transpose(0, 1)
-                ov = torch.bmm(o, w["w_uv"][:, c0:c1]) if ov is None else torch.baddbmm(ov, o, w["w_uv"][:, c0:c1])
-        return LO.heads_gate(ov, None)
+        return LO.heads_gate(LO.latent_attend(qf, pool, w["w_uv"], batch, H, R, rd, scale, 0), None)
 
     def _delta(self, li: int, h: torch.Tensor, batch: LO.RaggedBatch, cache: PagedStateCache) -> torch.Tensor:
         m, w = self.cfg.layers[li]["mixer"], self.w.layers[li]

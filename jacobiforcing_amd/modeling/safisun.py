@@ -26,6 +26,7 @@ from typing import Any, Dict, List, Optional, Tuple
 import torch
 import torch.nn.functional as F
 
+from . import read_tensors
 from .. import layer_ops as LO
 from ..engine.state_cache import PagedStateCache, RunSpec
 
@@ -201,16 +202,7 @@ class SafisunWeights:
 
     @classmethod
     def from_safetensors(cls, cfg: SafisunConfig, model_dir, device, dtype=torch.bfloat16) -> "SafisunWeights":
-        from safetensors import safe_open
-        files = sorted(Path(model_dir).glob("*.safetensors"))
-        if not files:
-            raise FileNotFoundError(f"no *.safetensors under {model_dir}")
-        tensors = {}
-        for f in files:
-            with safe_open(str(f), "pt", "cpu") as sf:
-                for k in sf.keys():
-                    tensors[k] = sf.get_tensor(k)
-        return cls(cfg, tensors, device, dtype)
+        return cls(cfg, read_tensors(model_dir), device, dtype)
 
     @classmethod
     def random(cls, cfg: SafisunConfig, device, dtype=torch.bfloat16, seed: int = 0) -> "SafisunWeights":
