@@ -1,9 +1,9 @@
 #!/usr/bin/env python3
-"""Prefill and decode throughput of a ragged model family (Lokizen, Vumalix, Bamanex, Mikipel, Safisun) at sizes that resemble a real model's
+"""Prefill and decode throughput of a ragged model family (Lokizen, Vumalix, Bamanex, Mikipel, Safisun, Voborax) at sizes that resemble a real model's
 layers, beside the package's closest existing model at equal width, depth, head sizes and active feed-forward width (Lokizen beside
-Qwen2; Vumalix, Bamanex, Mikipel and Safisun beside Lokizen and Qwen2) — random weights, synthetic tokens.
+Qwen2; Vumalix, Bamanex, Mikipel and Safisun beside Lokizen and Qwen2; Voborax beside Vumalix, Bamanex and Qwen2) — random weights, synthetic tokens.
 
-    python -m jacobiforcing_amd.drivers.ragged_bench [--design lokizen|vumalix|bamanex|mikipel|safisun] [--sizes small,medium] [--kernels]
+    python -m jacobiforcing_amd.drivers.ragged_bench [--design lokizen|vumalix|bamanex|mikipel|safisun|voborax] [--sizes small,medium] [--kernels]
     python bench.py --design lokizen            (the same, as one JSON line)
 
 Per size: prefill = whole prompts in one step (tokens / s), decode = one token for each of ``--decode-batch`` requests at a
@@ -649,97 +649,150 @@ def kernel_table_safisun(s, prompts, prompt_len, decode_batch, context, dtype=to
     return out
 
 
-def run_safisun(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
-    res = {"bench": "ragged_family", "design": "Safisun", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
-           "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
-    for name in sizes:
-        s = SIZES[name]
-        entry = {"shape": s, "safisun": bench_safisun(s, prompts, prompt_len, decode_batch, context)}
-        torch.cuda.empty_cache()
-        entry["lokizen"] = bench_lokizen(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        entry["qwen2"] = bench_qwen2(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        if kernels:
-            entry["kernels"] = kernel_table_safisun(s, prompts, prompt_len, decode_batch, context)
-            torch.cuda.empty_cache()
-        res["sizes"][name] = entry
-    return res
+# Voborax at Vumalix's widths, depths and latent sizes (Lokizen's experts): own latents under a window, borrowed latents, own latents without
+# positions, own latents under a window in turn; a dense feed-forward of the experts' active width, then experts with a quarter as many identity
+# experts beside them and a shared expert of one expert's width
+def voborax_config(s):
+    from ..modeling.voborax import VoboraxConfig
+    v = VSIZES["small" if s["width"] <= 1024 else "medium"]
+    moe = {"kind": "moe", "expert": {"ff": s["ff"]}, "router": {"experts": s["experts"], "identity": s["experts"] // 4, "top": s["top"]}, "shared": {"ff": s["ff"]}}
+    dense = {"kind": "dense", "ff": s["top"] * s["ff"]}
+    sizes = {"heads": v["lheads"], "dim": v["ldim"], "vdim": v["lvdim"], "kv_rank": v["kv_rank"], "q_rank": v["q_rank"]}
+    win = dict(sizes, rot_dim=v["rot"], rot={"dims": v["rot"], "base": 1e6}, scale=(v["ldim"] + v["rot"]) ** -0.5, mask={"size": v["window"]})
+    layers = []
+    for i in range(s["layers"]):
+        L = {"type": "latent_attention_2", "mixer": dict(sizes, scale=v["ldim"] ** -0.5)} if i % 4 == 2 else {"type": "latent_attention", "mixer": dict(win)}
+        if i % 4 == 1:
+            L["mixer"]["kv_from"] = i - 1
+        layers.append(dict(L, mlp=dense if i % 2 == 0 else moe))
+    return VoboraxConfig.from_dict({"architecture": "Voborax", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-5}, "embedding": {"scale": s["width"] ** 0.5},
+                                    "residual_mult": 0.5, "layers": layers})
 
 
-def run_mikipel(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
-    res = {"bench": "ragged_family", "design": "Mikipel", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
-           "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
-    for name in sizes:
-        s = SIZES[name]
-        entry = {"shape": s, "mikipel": bench_mikipel(s, prompts, prompt_len, decode_batch, context)}
-        torch.cuda.empty_cache()
-        entry["lokizen"] = bench_lokizen(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        entry["qwen2"] = bench_qwen2(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        if kernels:
-            entry["kernels"] = kernel_table_mikipel(s, prompts, prompt_len, decode_batch, context)
-            torch.cuda.empty_cache()
-        res["sizes"][name] = entry
-    return res
+def bench_voborax(s, prompts, prompt_len, decode_batch, context, dtype=torch.bfloat16):
+    from ..modeling.voborax import random_model
+    model = random_model(voborax_config(s), "cuda", dtype, max_positions=max(prompt_len, context) + 64)
+    return bench_ragged(model, s["vocab"], prompts, prompt_len, decode_batch, context)
 
 
-def run_bamanex(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
-    res = {"bench": "ragged_family", "design": "Bamanex", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
-           "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
-    for name in sizes:
-        s = SIZES[name]
-        entry = {"shape": s, "bamanex": bench_bamanex(s, prompts, prompt_len, decode_batch, context)}
-        torch.cuda.empty_cache()
-        entry["lokizen"] = bench_lokizen(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        entry["qwen2"] = bench_qwen2(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        if kernels:
-            entry["kernels"] = kernel_table_bamanex(s, prompts, prompt_len, decode_batch, context)
-            torch.cuda.empty_cache()
-        res["sizes"][name] = entry
-    return res
+def kernel_table_voborax(s, prompts, prompt_len, decode_batch, context, dtype=torch.bfloat16):
+    """Voborax's layer kernels alone at the size's shapes, prefill and decode, each beside the like kernel of the closest models at equal sizes
+    (Vumalix's output norm, latent stages and windowed latent attention; Mikipel's causal latent attention; Lokizen's update + norm over the
+    experts' rows; Bamanex's routed experts; Qwen2's SwiGLU launch)."""
+    from .. import layer_ops as LO
+    from .. import ops
+    dev = "cuda"
+    W, E, top, ff = s["width"], s["experts"], s["top"], s["ff"]
+    v = VSIZES["small" if W <= 1024 else "medium"]
+    H, D, rd, Dv, R, Rq, win = v["lheads"], v["ldim"], v["rot"], v["lvdim"], v["kv_rank"], v["q_rank"], v["window"]
+    ident = E // 4
+    page, es = 64, 2
+    per = -(-(max(prompt_len, context) + 1) // page)
+    slots = max(prompts, decode_batch)
+    tables = [list(range(b * per, (b + 1) * per)) for b in range(slots)]
+    g = torch.Generator().manual_seed(0)
+    rnd = lambda *sh: torch.randn(*sh, generator=g).to(dev).to(dtype)
+    lat, plain = rnd(slots * per * page, R + rd), rnd(slots * per * page, R)
+    a = torch.arange(max(prompt_len, context) + 8, dtype=torch.float32, device=dev).view(-1, 1) * torch.rand(rd // 2, device=dev).view(1, -1)
+    cos, sin = a.cos().contiguous(), a.sin().contiguous()
+    w_gu, w_down = rnd(E, 2 * ff, W) * 0.02, rnd(E, W, ff) * 0.02
+    w_uv, sink = rnd(H, R, Dv), torch.randn(H, device=dev)
+    corr = torch.randn(E + ident, generator=g).to(dev) * 0.01
+    out = {}
+
+    def row(name, secs, nbytes, flops, peak):
+        bound = max(nbytes / HBM_BPS, flops / peak)
+        out[name] = {"us": round(1e6 * secs, 1), "MB": round(nbytes / 1e6, 2), "GFLOP": round(flops / 1e9, 2), "roofline_fraction": round(bound / secs, 4)}
+
+    for phase, B, T, start in (("prefill", prompts, prompt_len, 0), ("decode", decode_batch, 1, context)):
+        n = B * T
+        batch = LO.RaggedBatch.build([T] * B, [start] * B, list(range(B)), tables[:B], page, dev)
+        causal = B * sum(start + t + 1 for t in range(T))                                       # visible (query, key) pairs per head
+        windowed = B * sum(min(start + t + 1, win) for t in range(T))
+        span_c, span_w = B * (start + T), B * min(start + T, win + T)                              # pool rows a launch has to read once
+        # output norm + update + the next sublayer's input  |  Vumalix: the same with one number for a weight, RMS
+        x, y, wf, one = torch.randn(n, W, device=dev), rnd(n, W), torch.randn(W, device=dev), torch.ones(1, device=dev)
+        row(f"{phase}.output_norm(one addend)", timed(lambda: LO.output_norm(x, [(y, None)], wf, 1e-5, LO.NORM_LAYER, 0.5, None, dtype)), n * W * (4 + 4 + es + es), 8.0 * n * W, VECTOR_FLOPS)
+        row(f"{phase}.vumalix.norm_add", timed(lambda: LO.norm_add(x, y, one, 1e-5, dtype)), n * W * (4 + 4 + es + es), 4.0 * n * W, VECTOR_FLOPS)
+        # the same over the experts' rows, a shared expert and identity choices  |  Lokizen: update + one norm over the experts' rows
+        h, z = rnd(n, W), torch.randn(n, E + ident, device=dev)
+        ye, ids, wts = LO.moe_experts(h, z, corr, top, 1.0, w_gu, w_down, route="softmax_renorm", renorm_eps=1e-20, gated=(LO.ACT_SILU, 0.0, 1.0, 0.0), identity=ident)
+        real = int((ids < E).sum())
+        row(f"{phase}.output_norm(experts, shared, identity)", timed(lambda: LO.output_norm(x, [(ye, None), (y, None)], wf, 1e-5, LO.NORM_LAYER, 0.5, None, dtype, choices=(ids, wts, E))),
+            n * W * (4 + 4 + es + es) + real * W * 4, (8.0 + 2 * top) * n * W, VECTOR_FLOPS)
+        ys, wb = torch.randn(n, top, W, device=dev), rnd(W)
+        row(f"{phase}.lokizen.add_rmsnorm(experts)", timed(lambda: LO.add_rmsnorm(x, ys, None, wb, 1e-5, dtype)), n * W * (4 + 4 * top + 4 + es), (4.0 + top) * n * W, VECTOR_FLOPS)
+        # latents: norms, rotation, append  |  Vumalix (halves for pairs)
+        pl = rnd(n, Rq + R + rd + H + (-(Rq + R + rd + H)) % 8)
+        wq, wk = rnd(Rq), rnd(R)
+        prep = lambda pool, pairing, r: LO.latent_prep(pl, 0, Rq, Rq, R, r, r, wq, wk, 1e-5, batch, cos, sin, pool, pairing=pairing)
+        row(f"{phase}.latent_prep", timed(lambda: prep(lat, LO.ROT_NEIGHBOURS, rd)), 2 * n * (Rq + R + rd) * es, 6.0 * n * (Rq + R + rd), VECTOR_FLOPS)
+        row(f"{phase}.latent_prep(no rotation)", timed(lambda: prep(plain, LO.ROT_NEIGHBOURS, 0)), 2 * n * (Rq + R) * es, 6.0 * n * (Rq + R), VECTOR_FLOPS)
+        row(f"{phase}.latent_prep(borrowed latents)", timed(lambda: prep(None, LO.ROT_NEIGHBOURS, rd)), 2 * n * Rq * es, 6.0 * n * Rq, VECTOR_FLOPS)
+        row(f"{phase}.vumalix.latent_prep", timed(lambda: prep(lat, LO.ROT_HALVES, rd)), 2 * n * (Rq + R + rd) * es, 6.0 * n * (Rq + R + rd), VECTOR_FLOPS)
+        qa, ql, qn = rnd(H, n, R), rnd(n, H * (D + rd)), rnd(n, H * D)
+        pack = lambda q, r, pairing: LO.latent_q_pack(qa, q, H, D, R, r, r, batch, cos, sin, pairing=pairing)
+        row(f"{phase}.latent_q_pack", timed(lambda: pack(ql, rd, LO.ROT_NEIGHBOURS)), 2 * n * H * (R + rd) * es, 6.0 * n * H * rd, VECTOR_FLOPS)
+        row(f"{phase}.latent_q_pack(no rotation)", timed(lambda: pack(qn, 0, LO.ROT_NEIGHBOURS)), 2 * n * H * R * es, 0.0, VECTOR_FLOPS)
+        row(f"{phase}.vumalix.latent_q_pack", timed(lambda: pack(ql, rd, LO.ROT_HALVES)), 2 * n * H * (R + rd) * es, 6.0 * n * H * rd, VECTOR_FLOPS)
+        # attention over the latents: window and head gate, causal with a sink  |  Vumalix: window; Mikipel: causal
+        qf, qc, gate = pack(ql, rd, LO.ROT_NEIGHBOURS), pack(qn, 0, LO.ROT_NEIGHBOURS), pl[:, Rq + R + rd:Rq + R + rd + H]
+        att = lambda q, pool, w, **kw: timed(lambda: LO.attn_sweep(q, pool, pool[:, :R], batch, H, 1, pool.shape[1], R, 0.1, w, **kw))
+        ab, af = span_w * (R + rd) * es + n * H * (2 * R + rd) * es, 2.0 * windowed * H * (2 * R + rd)
+        cb, cf = span_c * (R + rd) * es + n * H * (2 * R + rd) * es, 2.0 * causal * H * (2 * R + rd)
+        row(f"{phase}.attn_latent(window, head gate)", att(qf, lat, win, gate=gate, gate_per_head=True), ab, af, MATRIX_FLOPS)
+        row(f"{phase}.vumalix.attn_latent(window)", att(qf, lat, win), ab, af, MATRIX_FLOPS)
+        row(f"{phase}.attn_latent(causal, sink)", att(qc, plain, 0, sink=sink), span_c * R * es + 2 * n * H * R * es, 4.0 * causal * H * R, MATRIX_FLOPS)
+        row(f"{phase}.mikipel.attn_latent(causal)", att(qf, lat, 0), cb, cf, MATRIX_FLOPS)
+        ov, ge = rnd(H, n, Dv), rnd(n, H * Dv)
+        row(f"{phase}.heads_gate(none)", timed(lambda: LO.heads_gate(ov, None)), 2 * n * H * Dv * es, 0.0, VECTOR_FLOPS)
+        row(f"{phase}.vumalix.heads_gate", timed(lambda: LO.heads_gate(ov, ge)), 3 * n * H * Dv * es, 6.0 * n * H * Dv, VECTOR_FLOPS)
+        # activations  |  Qwen2's SwiGLU launch at the same widths
+        up, gu, g1 = rnd(n, top * ff), rnd(n, 2 * top * ff), rnd(n, 2 * ff)
+        row(f"{phase}.gated_act(gelu_tanh, no linear branch)", timed(lambda: LO.gated_act(up, 0, -1, top * ff, LO.ACT_GELU_TANH)), 2 * n * top * ff * es, 10.0 * n * top * ff, VECTOR_FLOPS)
+        row(f"{phase}.qwen2.swiglu", timed(lambda: ops.swiglu(gu)), 3 * n * top * ff * es, 4.0 * n * top * ff, VECTOR_FLOPS)
+        row(f"{phase}.gated_act(silu, shared width)", timed(lambda: LO.gated_act(g1, 0, ff, ff, LO.ACT_SILU)), 3 * n * ff * es, 6.0 * n * ff, VECTOR_FLOPS)
+        row(f"{phase}.qwen2.swiglu(shared width)", timed(lambda: ops.swiglu(g1)), 3 * n * ff * es, 4.0 * n * ff, VECTOR_FLOPS)
+        # routed experts: silu units, correction, identity experts  |  Bamanex: clamped units, no correction, none
+        used, usedb = len(set(ids[ids < E].tolist())), min(E, n * top)
+        t_moe = timed(lambda: LO.moe_experts(h, z, corr, top, 1.0, w_gu, w_down, route="softmax_renorm", renorm_eps=1e-20, gated=(LO.ACT_SILU, 0.0, 1.0, 0.0), identity=ident))
+        row(f"{phase}.moe_experts(identity experts)", t_moe, used * 3 * ff * W * es + n * W * es + real * W * 4, 6.0 * real * ff * W, MATRIX_FLOPS)
+        zb = z[:, :E].contiguous()
+        t_moe = timed(lambda: LO.moe_experts(h, zb, None, top, 1.0, w_gu, w_down, route="softmax_renorm", renorm_eps=1e-20, gated=(LO.ACT_CLAMPED_SWISH, 7.0, 1.702, 1.0)))
+        row(f"{phase}.bamanex.moe_experts", t_moe, usedb * 3 * ff * W * es + n * W * es + n * top * W * 4, 6.0 * n * top * ff * W, MATRIX_FLOPS)
+    return out
 
 
-def run_vumalix(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True):
-    res = {"bench": "ragged_family", "design": "Vumalix", "closest": "Lokizen", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
-           "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
-    for name in sizes:
-        s = VSIZES[name]
-        entry = {"shape": s, "vumalix": bench_vumalix(s, prompts, prompt_len, decode_batch, context)}
-        torch.cuda.empty_cache()
-        entry["lokizen"] = bench_lokizen(SIZES[name], prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        entry["qwen2"] = bench_qwen2(dict(SIZES[name], top=1, ff=s["ff"]), prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
-        if kernels:
-            entry["kernels"] = kernel_table_vumalix(s, prompts, prompt_len, decode_batch, context)
-            torch.cuda.empty_cache()
-        res["sizes"][name] = entry
-    return res
+# what a design's comparison runs at a size: the closest model, then (name, throughput function, shape) per model, then the kernel table
+def _comparison(design, name):
+    s, v = SIZES[name], VSIZES[name]
+    lok, qwen = ("lokizen", bench_lokizen, s), ("qwen2", bench_qwen2, s)
+    return {
+        "lokizen": ("Qwen2", [("lokizen", bench_lokizen, s), qwen], kernel_table),
+        "vumalix": ("Lokizen", [("vumalix", bench_vumalix, v), lok, ("qwen2", bench_qwen2, dict(s, top=1, ff=v["ff"]))], kernel_table_vumalix),
+        "bamanex": ("Lokizen", [("bamanex", bench_bamanex, s), lok, qwen], kernel_table_bamanex),
+        "mikipel": ("Lokizen", [("mikipel", bench_mikipel, s), lok, qwen], kernel_table_mikipel),
+        "safisun": ("Lokizen", [("safisun", bench_safisun, s), lok, qwen], kernel_table_safisun),
+        "voborax": ("Vumalix", [("voborax", bench_voborax, s), ("vumalix", bench_vumalix, v), ("bamanex", bench_bamanex, s), qwen], kernel_table_voborax),
+    }[design]
+
+
+DESIGNS = ("lokizen", "vumalix", "bamanex", "mikipel", "safisun", "voborax")
 
 
 def run(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, context=2048, kernels=True, design="lokizen"):
-    if design.lower() == "vumalix":
-        return run_vumalix(sizes, prompts, prompt_len, decode_batch, context, kernels)
-    if design.lower() == "bamanex":
-        return run_bamanex(sizes, prompts, prompt_len, decode_batch, context, kernels)
-    if design.lower() == "mikipel":
-        return run_mikipel(sizes, prompts, prompt_len, decode_batch, context, kernels)
-    if design.lower() == "safisun":
-        return run_safisun(sizes, prompts, prompt_len, decode_batch, context, kernels)
-    res = {"bench": "ragged_family", "design": "Lokizen", "closest": "Qwen2", "dtype": "bf16", "data": "synthetic", "prompts": prompts,
+    design = design.lower()
+    shape = (prompts, prompt_len, decode_batch, context)
+    res = {"bench": "ragged_family", "design": design.capitalize(), "closest": _comparison(design, sizes[0])[0], "dtype": "bf16", "data": "synthetic", "prompts": prompts,
            "prompt_len": prompt_len, "decode_batch": decode_batch, "context": context, "sizes": {}}
     for name in sizes:
-        s = SIZES[name]
-        entry = {"shape": s, "lokizen": bench_lokizen(s, prompts, prompt_len, decode_batch, context)}
-        torch.cuda.empty_cache()
-        entry["qwen2"] = bench_qwen2(s, prompts, prompt_len, decode_batch, context)
-        torch.cuda.empty_cache()
+        _, models, table = _comparison(design, name)
+        entry = {"shape": models[0][2]}
+        for key, fn, s in models:
+            entry[key] = fn(s, *shape)
+            torch.cuda.empty_cache()
         if kernels:
-            entry["kernels"] = kernel_table(s, prompts, prompt_len, decode_batch, context)
+            entry["kernels"] = table(models[0][2], *shape)
             torch.cuda.empty_cache()
         res["sizes"][name] = entry
     return res
@@ -747,7 +800,7 @@ def run(sizes=("small", "medium"), prompts=4, prompt_len=2048, decode_batch=32, 
 
 def main(argv=None):
     ap = argparse.ArgumentParser(description=__doc__.split("\n")[0])
-    ap.add_argument("--design", default="lokizen", choices=("lokizen", "vumalix", "bamanex", "mikipel", "safisun"))
+    ap.add_argument("--design", default="lokizen", choices=DESIGNS)
     ap.add_argument("--sizes", default="small,medium")
     ap.add_argument("--prompts", type=int, default=4)
     ap.add_argument("--prompt-len", type=int, default=2048)
