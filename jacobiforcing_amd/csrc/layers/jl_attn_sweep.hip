@@ -238,35 +238,35 @@ __global__ __launch_bounds__(AS_THREADS) void attn_sweep_kernel(jl_attn_args a, 
     }
 }
 
-// out[row] = sum_s part_s[row] * exp(m_s - M) / sum_s l_s * exp(m_s - M), in share order
+// out[row] = sum_s part_s[row] * exp(m_s - M) / sum_s l_s * exp(m_s - M), outputs summed in share order.  A workgroup joins AJ_ROWS of a
+// tile's rows; a row's weights are formed by one wavefront, lane s holding share s (at most 64).
+constexpr int AJ_ROWS = 4;
 __global__ __launch_bounds__(256) void attn_sweep_join_kernel(jl_attn_args a, int HF, int TQ, int HB) {
-    __shared__ float wS[AS_T * 64];                                 // [32][S] weight of every share of a row
-    const int H = a.H, Dv = a.Dv, S = a.splits, tid = threadIdx.x;
+    __shared__ float wS[AJ_ROWS * 64];
+    const int H = a.H, Dv = a.Dv, S = a.splits, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r0 = blockIdx.z * AJ_ROWS;
     const int *tile = a.tiles + 4 * (int64_t)blockIdx.x;
     const int cnt = tile[2], row0 = tile[3], per_group = H / a.G, c = blockIdx.y / HB;
     const int h0 = c * per_group + (blockIdx.y - c * HB) * HF, h_end = (c + 1) * per_group;
-    if (tile[0] < 0 || cnt <= 0) return;
+    if (tile[0] < 0 || r0 >= cnt * HF || r0 >= TQ * HF) return;
     const int64_t share = (int64_t)gridDim.x * gridDim.y * AS_T * (Dv + 2);
-    const float *base = a.scratch + ((int64_t)blockIdx.x * gridDim.y + blockIdx.y) * AS_T * (int64_t)(Dv + 2);
-    if (tid < AS_T) {
-        float M = -INFINITY, L = 0.f;
-        for (int sp = 0; sp < S; ++sp) M = fmaxf(M, base[sp * share + tid * (Dv + 2) + Dv]);
-        for (int sp = 0; sp < S; ++sp) {
-            const float m = base[sp * share + tid * (Dv + 2) + Dv];
-            const float w = m > -INFINITY ? __expf(m - M) : 0.f;
-            wS[tid * 64 + sp] = w;
-            L += w * base[sp * share + tid * (Dv + 2) + Dv + 1];
-        }
-        const float inv = L > 0.f ? 1.0f / L : 0.f;
-        for (int sp = 0; sp < S; ++sp) wS[tid * 64 + sp] *= inv;
+    const float *base = a.scratch + (((int64_t)blockIdx.x * gridDim.y + blockIdx.y) * AS_T + r0) * (int64_t)(Dv + 2);
+    for (int r = wave; r < AJ_ROWS; r += 4) {
+        const float *st = base + lane * share + r * (Dv + 2) + Dv;
+        const float m = lane < S ? st[0] : -INFINITY, l = lane < S ? st[1] : 0.f;
+        float M = m;
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) M = fmaxf(M, __shfl_xor(M, off, 64));
+        const float w = m > -INFINITY ? __expf(m - M) : 0.f;
+        const float L = wave_sum_f32(w * l);
+        wS[r * 64 + lane] = L > 0.f ? w / L : 0.f;
     }
     __syncthreads();
     bf16_t *out = (bf16_t *)a.out;
-    for (int e = tid; e < AS_T * Dv; e += 256) {
-        const int row = e / Dv, col = e - row * Dv, ii = row / HF, hh = h0 + row % HF;
+    for (int e = tid; e < AJ_ROWS * Dv; e += 256) {
+        const int r = e / Dv, col = e - r * Dv, row = r0 + r, ii = row / HF, hh = h0 + row % HF;
         if (row >= TQ * HF || ii >= cnt || hh >= h_end) continue;
         float v = 0.f;
-        for (int sp = 0; sp < S; ++sp) v += wS[row * 64 + sp] * base[sp * share + row * (Dv + 2) + col];
+        for (int sp = 0; sp < S; ++sp) v += wS[r * 64 + sp] * base[sp * share + r * (Dv + 2) + col];
         const int64_t o = (int64_t)(row0 + ii) * a.out_ld + hh * Dv + col;
         v *= a.out_scale;
         if (a.gate) v *= 1.0f / (1.0f + __expf(-ld_f((const bf16_t *)a.gate + (int64_t)(row0 + ii) * a.gate_ld + (a.gate_heads ? hh : hh * Dv + col))));
@@ -627,6 +627,6 @@ extern "C" int jl_attn_sweep(const jl_attn_args *ap, void *stream) {
         AS_CASE(1) AS_CASE(2) AS_CASE(3) AS_CASE(4)
     }
 #undef AS_CASE
-    if (a.splits > 1) attn_sweep_join_kernel<<<dim3(grid.x, grid.y), 256, 0, st>>>(a, hf, tq, hb);
+    if (a.splits > 1) attn_sweep_join_kernel<<<dim3(grid.x, grid.y, AS_T / AJ_ROWS), 256, 0, st>>>(a, hf, tq, hb);
     return jl_check_launch("attn_sweep_kernel");
 }

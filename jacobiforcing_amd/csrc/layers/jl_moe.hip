@@ -5,70 +5,71 @@
 #include "jl_common.h"
 #include <stdlib.h>
 
-// ---- router: one thread per token ------------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void moe_route_kernel(const float *__restrict__ logits, const float *__restrict__ correction, int64_t N,
-                                                         int E, int top, float scale, int32_t *__restrict__ ids,
-                                                         float *__restrict__ weights, int kind, float renorm_eps) {
-    const int64_t n = (int64_t)blockIdx.x * 256 + threadIdx.x;
+constexpr int MOE_MAX_E = 4096;   // experts (router outputs) at most
+
+// ---- router: one wavefront per token, NJ router outputs per lane (lane + 64 j) -------------------------------------------------------
+// Every lane keeps its outputs' comparison values and scores in registers; `top` rounds find the largest comparison value (ties: the lowest
+// index) by a butterfly over (value, index, score).  An output that was chosen leaves the race through a bit per lane and j.
+//   kind                      comparison value                       score
+//   JL_ROUTE_SIGMOID          sigmoid(z) + correction                sigmoid(z)
+//   JL_ROUTE_SOFTMAX_RENORM   softmax(z) + correction (none: z)      softmax(z), divided by the chosen scores' sum + renorm_eps
+//   JL_ROUTE_TOP_SOFTMAX      z                                      exp(z - the largest z), divided by the chosen ones' sum
+template <int NJ>
+__global__ __launch_bounds__(256) void moe_route_kernel(const float *__restrict__ logits, const float *__restrict__ correction, int64_t N, int E, int top,
+                                                         float scale, int32_t *__restrict__ ids, float *__restrict__ weights, int kind, float renorm_eps) {
+    const int64_t n = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
     if (n >= N) return;
     const float *z = logits + n * E;
-    if (kind == JL_ROUTE_TOP_SOFTMAX) {
-        // the largest `top` logits (ties: lowest index), found in descending order; weights = softmax over the chosen logits only
-        float zmax = 0.f, den = 0.f;
-        for (int s = 0; s < top; ++s) {
-            int best = -1;
-            float bz = 0.f;
-            for (int e = 0; e < E; ++e) {
-                bool taken = false;
-                for (int p = 0; p < s; ++p) taken |= ids[n * top + p] == e;
-                if (!taken && (best < 0 || z[e] > bz)) { best = e; bz = z[e]; }
-            }
-            if (s == 0) zmax = bz;
-            const float w = expf(bz - zmax);
-            ids[n * top + s] = best;
-            weights[n * top + s] = w;
-            den += w;
-        }
-        for (int s = 0; s < top; ++s) weights[n * top + s] = weights[n * top + s] / den * scale;
-        return;
+    float cmp[NJ], sc[NJ], zmax = -INFINITY;
+    uint64_t open = 0;                                              // bit j: this lane's output j exists and is not chosen yet
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+        const int e = lane + 64 * j;
+        cmp[j] = sc[j] = -INFINITY;
+        if (e < E) { cmp[j] = z[e]; open |= 1ull << j; zmax = fmaxf(zmax, cmp[j]); }
     }
-    if (kind == JL_ROUTE_SOFTMAX_RENORM) {
-        // scores = softmax over ALL experts; the largest `top` of score + correction (ties: lowest index); weights = score / (sum of the
-        // chosen scores + renorm_eps).  Without a correction the logits themselves are compared.
-        float zmax = -INFINITY, den = 0.f, chosen = 0.f;
-        for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, z[e]);
-        for (int e = 0; e < E; ++e) den += expf(z[e] - zmax);
-        for (int s = 0; s < top; ++s) {
-            int best = -1;
-            float bc = 0.f;
-            for (int e = 0; e < E; ++e) {
-                bool taken = false;
-                for (int p = 0; p < s; ++p) taken |= ids[n * top + p] == e;
-                const float ch = correction ? expf(z[e] - zmax) / den + correction[e] : z[e];
-                if (!taken && (best < 0 || ch > bc)) { best = e; bc = ch; }
-            }
-            const float sc = expf(z[best] - zmax) / den;
-            ids[n * top + s] = best;
-            weights[n * top + s] = sc;
-            chosen += sc;
-        }
-        for (int s = 0; s < top; ++s) weights[n * top + s] = weights[n * top + s] / (chosen + renorm_eps) * scale;
-        return;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) zmax = fmaxf(zmax, __shfl_xor(zmax, off, 64));
+    float den = 0.f;
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+        const int e = lane + 64 * j;
+        if (e >= E) continue;
+        sc[j] = kind == JL_ROUTE_SIGMOID ? 1.0f / (1.0f + expf(-cmp[j])) : expf(cmp[j] - zmax);
+        den += sc[j];
     }
+    if (kind == JL_ROUTE_SOFTMAX_RENORM) den = wave_sum_f32(den);
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+        const int e = lane + 64 * j;
+        if (e >= E) continue;
+        if (kind == JL_ROUTE_SOFTMAX_RENORM) sc[j] /= den;
+        if (kind == JL_ROUTE_SIGMOID) cmp[j] = sc[j];
+        if (kind == JL_ROUTE_SOFTMAX_RENORM && correction) cmp[j] = sc[j];
+        if (correction && kind != JL_ROUTE_TOP_SOFTMAX) cmp[j] += correction[e];
+    }
+    float chosen = 0.f;
     for (int s = 0; s < top; ++s) {
-        int best = -1;
-        float bc = 0.f, bs = 0.f;
-        for (int e = 0; e < E; ++e) {
-            bool taken = false;
-            for (int p = 0; p < s; ++p) taken |= ids[n * top + p] == e;
-            if (taken) continue;
-            const float sc = 1.0f / (1.0f + expf(-z[e]));
-            const float ch = sc + (correction ? correction[e] : 0.f);
-            if (best < 0 || ch > bc) { best = e; bc = ch; bs = sc; }
+        float bv = -INFINITY, bs = 0.f;
+        int be = 0x7fffffff;                                        // none
+#pragma unroll
+        for (int j = 0; j < NJ; ++j)
+            if ((open >> j & 1) && (be == 0x7fffffff || cmp[j] > bv)) { bv = cmp[j]; bs = sc[j]; be = lane + 64 * j; }
+#pragma unroll
+        for (int off = 32; off > 0; off >>= 1) {
+            const float ov = __shfl_xor(bv, off, 64), os = __shfl_xor(bs, off, 64);
+            const int oe = __shfl_xor(be, off, 64);
+            if (oe != 0x7fffffff && (be == 0x7fffffff || ov > bv || (!(bv > ov) && oe < be))) { bv = ov; bs = os; be = oe; }
         }
-        ids[n * top + s] = best;
-        weights[n * top + s] = bs * scale;
+        be = __shfl(be, 0, 64);                                     // one winner for all lanes, whatever the values compared to (not-a-numbers)
+        bs = __shfl(bs, 0, 64);
+        if ((be & 63) == lane) open &= ~(1ull << (be >> 6));
+        if ((s & 63) == lane) { ids[n * top + s] = be; weights[n * top + s] = bs; }
+        chosen += bs;
     }
+    const float by = kind == JL_ROUTE_SIGMOID ? 1.0f : kind == JL_ROUTE_SOFTMAX_RENORM ? chosen + renorm_eps : chosen;
+    for (int s = lane; s < top; s += 64) weights[n * top + s] = weights[n * top + s] / by * scale;      // what this lane wrote above
 }
 
 extern "C" int jl_moe_route(const float *logits, const float *correction, int64_t N, int32_t E, int32_t top, float scale, int32_t *ids,
@@ -76,8 +77,13 @@ extern "C" int jl_moe_route(const float *logits, const float *correction, int64_
     if (N <= 0) return JL_OK;
     if (!logits || !ids || !weights || E <= 0 || top <= 0 || top > E) return jl_fail(JL_E_INVALID, "jl_moe_route: null pointer or top > experts");
     if (kind < JL_ROUTE_SIGMOID || kind > JL_ROUTE_TOP_SOFTMAX) return jl_fail(JL_E_INVALID, "jl_moe_route: unknown kind %d", kind);
-    moe_route_kernel<<<dim3((unsigned)((N + 255) / 256)), 256, 0, (hipStream_t)stream>>>(logits, correction, N, E, top, scale, ids, weights, kind,
-                                                                                         renorm_eps);
+    if (E > MOE_MAX_E) return jl_fail(JL_E_INVALID, "jl_moe_route: at most %d router outputs", MOE_MAX_E);
+#define ROUTE_CASE(NJ) moe_route_kernel<NJ><<<dim3((unsigned)((N + 3) / 4)), 256, 0, (hipStream_t)stream>>>(logits, correction, N, E, top, scale, ids, weights, kind, renorm_eps)
+    if (E <= 64) ROUTE_CASE(1);
+    else if (E <= 256) ROUTE_CASE(4);
+    else if (E <= 1024) ROUTE_CASE(16);
+    else ROUTE_CASE(64);
+#undef ROUTE_CASE
     return jl_check_launch("moe_route_kernel");
 }
 
@@ -85,7 +91,6 @@ extern "C" int jl_moe_route(const float *logits, const float *correction, int64_
 constexpr int MOE_TM = 64;        // rows of a tile
 constexpr int MOE_TN = 64;        // output columns of a tile
 constexpr int MOE_TK = 32;        // depth of one LDS stage
-constexpr int MOE_MAX_E = 4096;
 
 __global__ __launch_bounds__(1024) void moe_group_kernel(const int32_t *__restrict__ ids, int64_t rows, int E, int tile_rows,
                                                           int32_t *__restrict__ perm, int32_t *__restrict__ offsets,

@@ -317,7 +317,7 @@ def test_embedding_with_a_rounded_copy():
     assert LO.embed_scale(e.cuda(), ids, 2.5, False)[1] is None and torch.equal(*LO.embed_scale(e.cuda(), ids, 2.5, True))
 
 
-ROUTED = [(5, 2, 3, 24), (1, 1, 1, 8), (7, 0, 2, 33), (3, 6, 9, 16), (16, 4, 4, 40), (2, 30, 5, 16)]
+ROUTED = [(5, 2, 3, 24), (1, 1, 1, 8), (7, 0, 2, 33), (3, 6, 9, 16), (16, 4, 4, 40), (2, 30, 5, 16), (70, 30, 66, 8), (2, 1100, 6, 8), (1, 4000, 3, 8)]
 
 
 @gpu
@@ -325,9 +325,9 @@ ROUTED = [(5, 2, 3, 24), (1, 1, 1, 8), (7, 0, 2, 33), (3, 6, 9, 16), (16, 4, 4, 
 @pytest.mark.parametrize("n", [1, 70, 300])
 def test_router_experts_and_identity_experts(E, ident, top, ff, n):
     """The router's choice with its correction, the grouped products over the experts that have weights, and the sum with the identity
-    experts' share inside the norm's launch."""
+    experts' share inside the norm's launch — up to thousands of router outputs (several per lane of the router's wavefront)."""
     from jacobiforcing_amd import layer_ops as LO
-    W = 48
+    W, n = 48, min(n, 20 if top > 60 else n)
     f = moe(E, ident, top, ff, 0)
     t = tensors_for(make_cfg([dict(win(), mlp=f)], width=W), 7)
     t["l0.mlp.correction"] = torch.randn(E + ident, generator=torch.Generator().manual_seed(2)) * 0.2
