@@ -1,7 +1,6 @@
-// jl_moe.hip — routed experts: the router's choice (sigmoid scores with a correction, a softmax renormalised over the chosen, or a
-// softmax over the chosen logits alone), the
-// rows grouped by expert, and the grouped products: up with relu^2 or plain (a gated unit's activation is its own launch), down with
-// the routing weights.
+// jl_moe.hip — routed experts: the router's choice (sigmoid scores with a correction, a softmax renormalised over the chosen with or without
+// a correction, or a softmax over the chosen logits alone), the rows grouped by expert (a choice of an expert without weights has none), and
+// the grouped products: up with relu^2, plain, or with the gated unit in its epilogue, down with the routing weights.
 #include "jl_common.h"
 #include <stdlib.h>
 
