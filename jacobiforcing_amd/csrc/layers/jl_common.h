@@ -76,19 +76,25 @@ __device__ __forceinline__ float soft_cap_small(float s, float inv_cap) {
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 // gated units of a feed-forward (jl_gated_act, and the grouped product that applies them in its epilogue)
+// FAST: the sigmoid on the hardware's exponential and reciprocal (a few 1e-7 off), for results that are rounded to bfloat16
+template <bool FAST = false> __device__ __forceinline__ float sigmoid_f(float z) {
+    if (FAST) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.44269504f * z));
+    return 1.0f / (1.0f + expf(-z));
+}
 // 0.5 z (1 + tanh(u)) = z sigmoid(2u), u = sqrt(2/pi) (z + 0.044715 z^3)
-__device__ __forceinline__ float gelu_tanh_f(float z) {
-    return z / (1.0f + expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+template <bool FAST = false> __device__ __forceinline__ float gelu_tanh_f(float z) {
+    return z * sigmoid_f<FAST>(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
 __device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
+template <bool FAST = false> __device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f<FAST>(z); }
+template <bool FAST = false>
 __device__ __forceinline__ float gated_unit_f(float g, float u, int kind, float limit, float alpha, float shift) {
-    if (kind == JL_ACT_GELU_TANH) return gelu_tanh_f(g) * u;
-    if (kind == JL_ACT_SILU) return silu_f(g) * u;
+    if (kind == JL_ACT_GELU_TANH) return gelu_tanh_f<FAST>(g) * u;
+    if (kind == JL_ACT_SILU) return silu_f<FAST>(g) * u;
     if (kind == JL_ACT_GELU_ERF) return gelu_erf_f(g) * u;
     g = fminf(g, limit);                                            // clamped swish: the gate capped from above, the linear branch from both sides
     u = fminf(fmaxf(u, -limit), limit);
-    return g / (1.0f + expf(-alpha * g)) * (u + shift);
+    return g * sigmoid_f<FAST>(alpha * g) * (u + shift);
 }
 
 #define JL_DISPATCH(dtype, ...)                                   \

@@ -301,7 +301,7 @@ __global__ __launch_bounds__(256) void moe_gemm_mfma_kernel(const bf16_t *__rest
             const float c = half ? acc1[i] : acc0[i];
             const int r = r0 + m;
             if (GATED) {
-                st_f((bf16_t *)out + (int64_t)r * n_out + n, gated_unit_f(c, half ? acu1[i] : acu0[i], act.kind, act.limit, act.alpha, act.shift));
+                st_f((bf16_t *)out + (int64_t)r * n_out + n, gated_unit_f<true>(c, half ? acu1[i] : acu0[i], act.kind, act.limit, act.alpha, act.shift));
             } else if (mode == JL_MOE_UP_PLAIN) {
                 st_f((bf16_t *)out + (int64_t)r * n_out + n, c);
             } else if (mode == 0) {

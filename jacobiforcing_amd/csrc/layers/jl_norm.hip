@@ -146,8 +146,9 @@ __global__ __launch_bounds__(256) void gated_act_vec_kernel(const T *__restrict_
     constexpr int VEC = 16 / sizeof(T);
     const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (e >= vecs) return;
+    constexpr bool FAST = sizeof(T) == 2;
     const int per_row = F / VEC;
-    const int64_t n = e / per_row;
+    const int64_t n = vecs <= 0xffffffffll ? (int64_t)((uint32_t)e / (uint32_t)per_row) : e / per_row;      // a 64-bit division costs as much as the unit
     const int c = (int)(e - n * per_row) * VEC;
     float g[VEC], u[VEC];
     ld16(z + n * ld + g_col + c, g);
@@ -157,7 +158,7 @@ __global__ __launch_bounds__(256) void gated_act_vec_kernel(const T *__restrict_
         for (int i = 0; i < VEC; ++i) u[i] = 1.0f;
     const float rg = row_gate ? 1.0f / (1.0f + expf(-ld_f(row_gate + n * rg_ld))) : 1.0f;
 #pragma unroll
-    for (int i = 0; i < VEC; ++i) g[i] = gated_unit_f(g[i], u[i], kind, limit, alpha, shift) * rg;
+    for (int i = 0; i < VEC; ++i) g[i] = gated_unit_f<FAST>(g[i], u[i], kind, limit, alpha, shift) * rg;
     st16(out + n * F + c, g);
 }
 

@@ -445,6 +445,37 @@ def test_attention_over_the_latents_at_every_kind_of_size(H, R, rd, window):
             assert rel_err(got[:, -1], want[:, -1]) < 2 * tol
 
 
+@gpu
+@pytest.mark.parametrize("H,R,rd", [(16, 64, 16), (12, 128, 32), (40, 96, 0)])
+@pytest.mark.parametrize("window", [0, 90])
+def test_long_portions_take_the_wide_tiles(H, R, rd, window):
+    """Hundreds of tokens per request in bfloat16: the 128-row form of the one-sweep kernel over the latents, with sink and gate, beside a portion
+    that starts inside a sequence."""
+    from jacobiforcing_amd import layer_ops as LO
+    g = torch.Generator().manual_seed(H)
+    page, Dv, scale, bf = 64, 8, 0.9 / (R + rd) ** 0.5, torch.bfloat16
+    starts, counts = [0, 300], [700, 410]
+    tables = [list(range(12))[::-1], list(range(12, 24))]
+    pool, q = torch.randn(24 * page, R + rd, generator=g).to(bf), torch.randn(sum(counts), H * (R + rd), generator=g).to(bf)
+    gate, sink, w_uv = torch.randn(sum(counts), H, generator=g).to(bf), torch.randn(H, generator=g) + 3, (torch.randn(H, R, Dv, generator=g) * R ** -0.5).to(bf)
+    b = LO.RaggedBatch.build(counts, starts, [0, 1], tables, page, "cuda")
+    tq = LO.attn_sweep_tile_rows(bf, H, 1, R + rd, R, pool.cuda(), pool.cuda()[:, :R])
+    assert b.tiles(tq).shape[0] * -(-H // 32) >= LO.SWEEP_SPLIT_BELOW_GROUPS                        # what makes the launch choose the wide form
+    got = LO.latent_attend(q.cuda(), pool.cuda(), w_uv.cuda(), b, H, R, rd, scale, window, sink=sink.cuda(), gate=gate.cuda()).float().cpu()
+    r = 0
+    for bb in range(2):
+        n, T = counts[bb], starts[bb] + counts[bb]
+        kv = pool[torch.tensor([tables[bb][p // page] * page + p % page for p in range(T)])].double()
+        s = torch.einsum("ihd,jd->hij", q[r:r + n].double().view(n, H, R + rd), kv) * scale
+        w = O.masked_softmax(s, O.visible(T, window or None)[starts[bb]:], sink.double())
+        o = torch.einsum("hij,jr->hir", w, kv[:, :R]) * torch.sigmoid(gate[r:r + n].double()).T.unsqueeze(-1)
+        want = torch.bmm(o, w_uv.double())
+        assert rel_err(got[:, r:r + n], want) < 2e-2
+        err = ((got[:, r:r + n].double() - want) ** 2).mean((0, 2)).sqrt() / (want ** 2).mean((0, 2)).sqrt()
+        assert float(err.max()) < 6e-2
+        r += n
+
+
 MIXER_SIZES = [win(), win(1, 20, 6, 10, 33, 17, 1), win(5, 12, 2, 16, 40, 44, 9), win(8, 32, 32, 32, 64, 96, 30, 1e4, 0.125), win(16, 64, 16, 64, 128, 64, 64, scale=0.1),
                win(2, 8, 24, 40, 96, 20, 33), win(3, 16, 16, 8, 144, 24, 70, scale=0.2), win(12, 48, 64, 48, 512, 160, 50, scale=0.1),
                cau(), cau(1, 8, 8, 20, 12), cau(7, 10, 6, 33, 15), cau(8, 32, 48, 64, 96), cau(12, 64, 32, 96, 80, 0.12), cau(20, 16, 16, 200, 40), cau(33, 8, 8, 32, 24)]
